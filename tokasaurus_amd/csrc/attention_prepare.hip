@@ -16,7 +16,8 @@
 // elements behind them (a latent beside a rotated key part that is no part of it).  `vfreq`: the values
 // are turned too, every element of a head, pair m by position * vfreq[m], pairs (m, m + dv/2) with
 // `v_pair_half` and (2m, 2m + 1) without.  `rot_scale`: cosine and sine of the queries' and keys'
-// rotation are both multiplied by it (1: a plain rotation).
+// rotation are both multiplied by it (1: a plain rotation).  `rotate_q` 0: only the keys are turned (a query row that
+// is not yet the heads' queries but a latent they are made from).
 // The arithmetic is 32-bit from the product's rounded output to the one rounding at the store.
 //   row: [nq*dq | nkv*dk | nkv*dv]  (only the first part when !write_cache; no third part with v_from_k)
 //   K pages: [page][kv head][dk / 8][P][8]    V pages: [page][kv head][P / 4][dv][4]
@@ -49,7 +50,7 @@ __global__ __launch_bounds__(256) void qk_prepare_kernel(
     const float* __restrict__ q_weight, const float* __restrict__ k_weight, float eps,
     const float* __restrict__ freq, T* __restrict__ kcache, T* __restrict__ vcache, int nq, int nkv,
     int dq, int dk, int dv, int rot, int P, int write_cache, int pair_half, int v_from_k, int per_head, int k_skip,
-    const float* __restrict__ vfreq, int v_pair_half, float rot_scale) {
+    const float* __restrict__ vfreq, int v_pair_half, float rot_scale, int rotate_q) {
   extern __shared__ float cs[];  // [rot / 2] cosines, [rot / 2] sines, then (vfreq) [dv / 2] cosines, [dv / 2] sines, then (per_head) [nq + nkv] factors
   __shared__ float red[16];
   const int t = blockIdx.x;
@@ -113,9 +114,10 @@ __global__ __launch_bounds__(256) void qk_prepare_kernel(
   __syncthreads();  // the table of this token's angles is written
 
   // queries, in place, a pair a thread (a head of odd size ends in a single element)
-  const int hq = pair_items(dq, rot, pair_half);
+  const int q_rot = rotate_q ? rot : 0;
+  const int hq = pair_items(dq, q_rot, pair_half);
   for (int i = threadIdx.x; i < nq * hq; i += blockDim.x) {
-    const PairItem it = pair_item(i % hq, dq, rot, pair_half);
+    const PairItem it = pair_item(i % hq, dq, q_rot, pair_half);
     const int x0 = (i / hq) * dq + it.e0, x1 = (i / hq) * dq + it.e1;
     if (per_head) rq = head_r[i / hq];
     float u = to_f32<T>(row[x0]) * rq, v = it.two ? to_f32<T>(row[x1]) * rq : 0.f;
@@ -186,10 +188,10 @@ TK_API int tk_qk_prepare(int dt, void* qkv, int row_stride, const int* positions
                          const float* k_weight, float eps, const float* freq, void* kcache, void* vcache,
                          int n_tokens, int nq, int nkv, int dq, int dk, int dv, int rot, int P, int write_cache,
                          int pair_half, int v_from_k, int per_head, int k_skip, const float* vfreq, int v_pair_half,
-                         float rot_scale, hipStream_t stream) {
+                         float rot_scale, int rotate_q, hipStream_t stream) {
   TK_REQUIRE(n_tokens >= 0 && nq >= 0 && nkv >= 0 && nq + nkv > 0 && dq > 0 && dk > 0 && dv > 0 && P > 0,
              "qk_prepare: bad sizes tokens=%d nq=%d nkv=%d dq=%d dk=%d dv=%d P=%d", n_tokens, nq, nkv, dq, dk, dv, P);
-  TK_REQUIRE(rot >= 0 && rot <= dk && rot <= dq && rot % 2 == 0, "qk_prepare: %d rotated elements of heads of %d and %d", rot, dq, dk);
+  TK_REQUIRE(rot >= 0 && rot <= dk && (rot <= dq || !rotate_q) && rot % 2 == 0, "qk_prepare: %d rotated elements of heads of %d and %d", rot, dq, dk);
   TK_REQUIRE(rot == 0 || freq, "qk_prepare: a rotation needs its frequencies");
   TK_REQUIRE(k_skip >= 0 && k_skip % 2 == 0 && k_skip < dk && (k_skip == 0 || !pair_half || k_skip == rot),
              "qk_prepare: %d leading elements of a key of %d left out of its norm", k_skip, dk);
@@ -205,12 +207,12 @@ TK_API int tk_qk_prepare(int dt, void* qkv, int row_stride, const int* positions
     hipLaunchKernelGGL(qk_prepare_kernel<float>, dim3(n_tokens), dim3(256), smem, stream, (float*)qkv,
                        row_stride, positions, token_req, block_table, table_stride, q_weight, k_weight, eps,
                        freq, (float*)kcache, (float*)vcache, nq, nkv, dq, dk, dv, rot, P, write_cache, pair_half, v_from_k,
-                       per_head, k_skip, vfreq, v_pair_half, rot_scale);
+                       per_head, k_skip, vfreq, v_pair_half, rot_scale, rotate_q);
   else
     hipLaunchKernelGGL(qk_prepare_kernel<bf16_t>, dim3(n_tokens), dim3(256), smem, stream, (bf16_t*)qkv,
                        row_stride, positions, token_req, block_table, table_stride, q_weight, k_weight, eps,
                        freq, (bf16_t*)kcache, (bf16_t*)vcache, nq, nkv, dq, dk, dv, rot, P, write_cache, pair_half, v_from_k,
-                       per_head, k_skip, vfreq, v_pair_half, rot_scale);
+                       per_head, k_skip, vfreq, v_pair_half, rot_scale, rotate_q);
   TK_CHECK_LAUNCH("qk_prepare");
   return 0;
 }
@@ -306,5 +308,52 @@ TK_API int tk_unrotate_gate(int dt, void* o, int o_stride, const int* positions,
     hipLaunchKernelGGL(unrotate_gate_kernel<bf16_t>, dim3(n_tokens), dim3(256), smem, stream, (bf16_t*)o, o_stride, positions, vfreq,
                        pair_half, (const bf16_t*)gate, gate_stride, nq, dv);
   TK_CHECK_LAUNCH("unrotate_gate");
+  return 0;
+}
+
+// --------------------------------------------------------------------------
+// In place: the leading `rot` elements of every head of a token's row [heads][d] turned by position * freq[i], pairs
+// (i, i + rot/2) with `pair_half` and (2i, 2i + 1) without; the rest of a head is not touched.  For queries whose
+// projection reads a latent that another kernel has normed.  A workgroup a token, 32-bit arithmetic, one rounding.
+// --------------------------------------------------------------------------
+template <typename T>
+__global__ __launch_bounds__(256) void rotate_heads_kernel(T* __restrict__ x, int stride, const int* __restrict__ positions,
+                                                           const float* __restrict__ freq, int heads, int d, int rot, int pair_half,
+                                                           float rot_scale) {
+  extern __shared__ float cs[];  // [rot / 2] cosines, [rot / 2] sines
+  const int t = blockIdx.x, half = rot / 2;
+  const float pos = (float)positions[t];
+  for (int i = threadIdx.x; i < half; i += blockDim.x) {
+    float s, c;
+    sincosf(__fmul_rn(pos, freq[i]), &s, &c);
+    cs[i] = c * rot_scale;
+    cs[half + i] = s * rot_scale;
+  }
+  __syncthreads();
+  T* row = x + (size_t)t * stride;
+  for (int i = threadIdx.x; i < heads * half; i += blockDim.x) {
+    const int h = i / half, m = i % half;
+    T* e0 = row + (size_t)h * d + (pair_half ? m : 2 * m);
+    T* e1 = e0 + (pair_half ? half : 1);
+    float u = to_f32<T>(*e0), v = to_f32<T>(*e1);
+    rotate_pair(u, v, cs[m], cs[half + m], u, v);
+    *e0 = from_f32<T>(u);
+    *e1 = from_f32<T>(v);
+  }
+}
+
+TK_API int tk_rotate_heads(int dt, void* x, int stride, const int* positions, const float* freq, int n_tokens, int heads, int d,
+                           int rot, int pair_half, float rot_scale, hipStream_t stream) {
+  TK_REQUIRE(x && positions && freq && n_tokens >= 0 && heads > 0 && rot > 0 && rot % 2 == 0 && rot <= d && rot <= 8192 && stride >= heads * d,
+             "rotate_heads: bad sizes tokens=%d heads=%d d=%d rot=%d or a pointer is missing", n_tokens, heads, d, rot);
+  if (n_tokens == 0) return 0;
+  const size_t smem = sizeof(float) * (size_t)rot;
+  if (dt == TK_F32)
+    hipLaunchKernelGGL(rotate_heads_kernel<float>, dim3(n_tokens), dim3(256), smem, stream, (float*)x, stride, positions, freq, heads, d,
+                       rot, pair_half, rot_scale);
+  else
+    hipLaunchKernelGGL(rotate_heads_kernel<bf16_t>, dim3(n_tokens), dim3(256), smem, stream, (bf16_t*)x, stride, positions, freq, heads,
+                       d, rot, pair_half, rot_scale);
+  TK_CHECK_LAUNCH("rotate_heads");
   return 0;
 }

@@ -42,6 +42,8 @@ struct GroupedArgs {
   void* C;
   int ldc;
   int N, K, slots;
+  const float* row_scale;  // (gated form) a factor on a slot's sums of gate and up alike, row_scale[scale_row[slot]]; null: none
+  const int* scale_row;
 };
 
 // NT: blocks of 16 outputs a wavefront; GLU: the gated form; F32: 32-bit output
@@ -115,12 +117,13 @@ __global__ __launch_bounds__(GG_WAVES * TK_WAVE) void grouped_gemm_kernel(Groupe
     if (a.a_row && a.a_row[slot] < 0) continue;
     const int crow = a.c_row ? a.c_row[slot] : slot;
     if (crow < 0) continue;
+    const float f = GLU && a.row_scale ? a.row_scale[a.scale_row[slot]] : 1.f;  // (a slot that is filled names its row)
 #pragma unroll
     for (int t = 0; t < NT; ++t) {
       const int n = n0 + t * 16 + 4 * q;
       float y[4];
 #pragma unroll
-      for (int j = 0; j < 4; ++j) y[j] = GLU ? silu_mul_bf16(acc[t][mb][j], acc[t + (GLU ? NT : 0)][mb][j]) : acc[t][mb][j];
+      for (int j = 0; j < 4; ++j) y[j] = GLU ? silu_mul_bf16(acc[t][mb][j] * f, acc[t + (GLU ? NT : 0)][mb][j] * f) : acc[t][mb][j];
       const size_t at = (size_t)crow * a.ldc + (size_t)g * a.c_cols + n;
 #pragma unroll
       for (int j = 0; j < 4; ++j) {
@@ -135,14 +138,17 @@ __global__ __launch_bounds__(GG_WAVES * TK_WAVE) void grouped_gemm_kernel(Groupe
 
 TK_API int tk_grouped_gemm_bf16(const void* A, int lda, const int* a_row, const int* c_row, const int* tile_group, int tiles,
                                 int groups_z, int a_cols, int c_cols, const void* W, size_t w_stride, void* C, int ldc,
-                                int N, int K, int slots, int glu, int out_f32, hipStream_t stream) {
+                                int N, int K, int slots, int glu, int out_f32, const float* row_scale, const int* scale_row,
+                                hipStream_t stream) {
   TK_REQUIRE(A && W && C && N > 0 && K > 0 && slots >= 0 && tiles >= 0, "grouped_gemm: bad arguments");
   TK_REQUIRE(K % 8 == 0 && lda % 8 == 0 && a_cols % 8 == 0 && w_stride % 8 == 0 && (((uintptr_t)A | (uintptr_t)W) & 15) == 0,
              "grouped_gemm: rows of A and W must start at multiples of 16 bytes (K=%d lda=%d)", K, lda);
   TK_REQUIRE((tile_group != nullptr) != (groups_z > 0), "grouped_gemm: groups come by tile or by the grid, not both");
+  TK_REQUIRE(!row_scale || (glu && scale_row && a_row), "grouped_gemm: a factor a row goes with the gated form and rows by slot");
   TK_REQUIRE(!(glu && out_f32), "grouped_gemm: the gated form writes the storage type");
   if (tiles == 0 || slots == 0) return 0;
-  GroupedArgs a{(const bf16_t*)A, lda, a_row, c_row, tile_group, a_cols, c_cols, (const bf16_t*)W, w_stride, C, ldc, N, K, slots};
+  GroupedArgs a{(const bf16_t*)A, lda, a_row, c_row, tile_group, a_cols, c_cols, (const bf16_t*)W, w_stride, C, ldc, N, K, slots,
+                row_scale, scale_row};
   const int nt = glu ? 2 : 4;
   const dim3 grid(tiles, (N + GG_WAVES * nt * 16 - 1) / (GG_WAVES * nt * 16), groups_z > 0 ? groups_z : 1);
   TK_REQUIRE(grid.y < 65536 && grid.z < 65536, "grouped_gemm: too many outputs or groups");
@@ -215,11 +221,12 @@ TK_API int tk_expert_sort(const int* ids, int pairs, int top, int experts, int m
 // --------------------------------------------------------------------------
 // out[t, c] = sum over the places k of token t, in order, of weights[t, k] * (y[t * top + k, c] for a routed expert,
 // h[t, c] for an identity expert), plus shared_gate[t] * shared[t, c].  y: [pairs, width] in the storage type.
+// `unit` != 0: a routed expert's row is added as it is.
 // --------------------------------------------------------------------------
 __global__ __launch_bounds__(256) void expert_sum_kernel(const bf16_t* __restrict__ h, int h_stride, const bf16_t* __restrict__ y,
                                                          const int* __restrict__ ids, const float* __restrict__ weights,
                                                          const float* __restrict__ shared, const float* __restrict__ shared_gate,
-                                                         float* __restrict__ out, int width, int experts, int top) {
+                                                         float* __restrict__ out, int width, int experts, int top, int unit) {
   const int t = blockIdx.x;
   for (int c = threadIdx.x; c < width; c += blockDim.x) {
     float acc = 0.f;
@@ -227,7 +234,7 @@ __global__ __launch_bounds__(256) void expert_sum_kernel(const bf16_t* __restric
       const int e = ids[(size_t)t * top + k];
       if (e < 0) continue;
       const float v = e < experts ? __bfloat162float(y[((size_t)t * top + k) * width + c]) : __bfloat162float(h[(size_t)t * h_stride + c]);
-      acc = fmaf(weights[(size_t)t * top + k], v, acc);
+      acc = fmaf(unit && e < experts ? 1.f : weights[(size_t)t * top + k], v, acc);
     }
     if (shared) acc = fmaf(shared_gate[t], shared[(size_t)t * width + c], acc);
     out[(size_t)t * width + c] = acc;
@@ -235,12 +242,12 @@ __global__ __launch_bounds__(256) void expert_sum_kernel(const bf16_t* __restric
 }
 
 TK_API int tk_expert_sum(const void* h, int h_stride, const void* y, const int* ids, const float* weights, const float* shared,
-                         const float* shared_gate, float* out, int tokens, int width, int experts, int top, hipStream_t stream) {
+                         const float* shared_gate, float* out, int tokens, int width, int experts, int top, int unit, hipStream_t stream) {
   TK_REQUIRE(h && y && ids && weights && out && (!shared || shared_gate) && tokens >= 0 && width > 0 && top > 0 && h_stride >= width,
              "expert_sum: bad arguments");
   if (tokens == 0) return 0;
   hipLaunchKernelGGL(expert_sum_kernel, dim3(tokens), dim3(256), 0, stream, (const bf16_t*)h, h_stride, (const bf16_t*)y, ids,
-                     weights, shared, shared_gate, out, width, experts, top);
+                     weights, shared, shared_gate, out, width, experts, top, unit);
   TK_CHECK_LAUNCH("expert_sum");
   return 0;
 }

@@ -2,10 +2,10 @@
 // per-head products of a mixer whose heads share a latent.  T is the storage type of weights
 // and activations; sums are 32-bit, and the router is 32-bit arithmetic throughout.
 //
-//   tk_expert_route      per token: logits over all experts, softmax, choice by score + correction
-//                        inside the best groups of neighbouring experts, the chosen experts'
-//                        scores as weights; optionally the sigmoid gate of a shared expert
-//   tk_expert_gate_up    per (token, chosen expert): act(W_gate h) * (W_up h)
+//   tk_expert_route      per token: logits over all experts, their softmax or sigmoids, choice by score
+//                        (+ correction) inside the best groups of neighbouring experts, the chosen
+//                        experts' scores as weights; optionally the sigmoid gate of a shared expert
+//   tk_expert_gate_up    per (token, chosen expert): act(W_gate h) * (W_up h), of h or of weight * h
 //   tk_expert_combine    per token: sum of weight * W_down(...) over its experts, weight * h for an
 //                        identity expert, plus gate * (a shared expert's output)
 //   tk_head_linear       y[t, h, :] = W[h] x[t, h, :]: one matrix a head
@@ -69,11 +69,12 @@ __device__ __forceinline__ void wave_dot2(const T* __restrict__ w0, const T* __r
 
 // --------------------------------------------------------------------------
 // The router.  One workgroup a token.  n_all = routed + identity experts.  ids [tokens, top] names
-// the chosen experts in the order of their choice scores, weights [tokens, top] their softmax
-// scores (the correction moves the choice, not the weight); with `norm_scale` != 0 the chosen scores divided by
+// the chosen experts in the order of their choice scores, weights [tokens, top] their scores: softmax, or
+// SIGMOID, each the sigmoid of its own logit (the correction, where there is one, moves the choice, not the weight;
+// without one sigmoid scores are ranked by their logits, which order them without saturating); with `norm_scale` != 0 the chosen scores divided by
 // their sum (+ 1e-20) and multiplied by norm_scale.  Without `w_gate` a given `shared_gate` is filled with ones.
 // --------------------------------------------------------------------------
-template <typename T>
+template <typename T, bool SIGMOID>
 __global__ __launch_bounds__(1024) void expert_route_kernel(
     const T* __restrict__ h, int h_stride, const T* __restrict__ w_router, const float* __restrict__ correction,
     const T* __restrict__ w_gate, int width, int n_all, int groups, int keep, int top, int* __restrict__ ids,
@@ -96,7 +97,13 @@ __global__ __launch_bounds__(1024) void expert_route_kernel(
   __syncthreads();
   // the rest is the work of one wavefront; the others only keep the barriers
   const bool on = wave == 0;
-  if (on) {
+  if (on && SIGMOID) {
+    for (int e = lane; e < n_all; e += TK_WAVE) {
+      const float z = score[e], s = 1.0f / (1.0f + expf(-z));
+      score[e] = s;
+      choice[e] = correction ? s + correction[e] : z;
+    }
+  } else if (on) {
     float m = -INFINITY;
     for (int e = lane; e < n_all; e += TK_WAVE) m = fmaxf(m, score[e]);
     m = wave_max(m);
@@ -110,7 +117,7 @@ __global__ __launch_bounds__(1024) void expert_route_kernel(
     for (int e = lane; e < n_all; e += TK_WAVE) {
       const float s = score[e] / sum;
       score[e] = s;
-      choice[e] = s + correction[e];
+      choice[e] = correction ? s + correction[e] : s;
     }
   }
   __syncthreads();
@@ -163,40 +170,43 @@ __global__ __launch_bounds__(1024) void expert_route_kernel(
 
 TK_API int tk_expert_route(int dt, const void* h, int h_stride, const void* w_router, const float* correction,
                            const void* w_gate, int tokens, int width, int n_all, int groups, int keep, int top,
-                           int* ids, float* weights, float* shared_gate, float norm_scale, hipStream_t stream) {
+                           int* ids, float* weights, float* shared_gate, float norm_scale, int sigmoid, hipStream_t stream) {
   TK_REQUIRE(tokens >= 0 && width > 0 && n_all > 0 && groups > 0 && n_all % groups == 0 && keep > 0 && keep <= groups &&
                  top > 0 && top <= n_all,
              "expert_route: bad sizes tokens=%d width=%d experts=%d groups=%d keep=%d top=%d", tokens, width, n_all,
              groups, keep, top);
-  TK_REQUIRE(h && w_router && correction && ids && weights && (!w_gate || shared_gate) && h_stride >= width,
+  TK_REQUIRE(h && w_router && ids && weights && (!w_gate || shared_gate) && h_stride >= width,
              "expert_route: a pointer is missing or the row stride is too short");
   const size_t smem = sizeof(float) * (size_t)(2 * n_all + groups);
   TK_REQUIRE(smem <= 48 * 1024, "expert_route: %d experts do not fit the local memory", n_all);
   if (tokens == 0) return 0;
   // a wavefront a logit where the step has few tokens (each dot product is a chain of loads), four wavefronts for many
   const int threads = tokens <= 64 ? 1024 : 256;
-  if (dt == TK_F32)
-    hipLaunchKernelGGL(expert_route_kernel<float>, dim3(tokens), dim3(threads), smem, stream, (const float*)h, h_stride,
-                       (const float*)w_router, correction, (const float*)w_gate, width, n_all, groups, keep, top, ids,
-                       weights, shared_gate, norm_scale);
-  else
-    hipLaunchKernelGGL(expert_route_kernel<bf16_t>, dim3(tokens), dim3(threads), smem, stream, (const bf16_t*)h, h_stride,
-                       (const bf16_t*)w_router, correction, (const bf16_t*)w_gate, width, n_all, groups, keep, top, ids,
-                       weights, shared_gate, norm_scale);
+#define ER_LAUNCH(T, S)                                                                                                       \
+  hipLaunchKernelGGL((expert_route_kernel<T, S>), dim3(tokens), dim3(threads), smem, stream, (const T*)h, h_stride,            \
+                     (const T*)w_router, correction, (const T*)w_gate, width, n_all, groups, keep, top, ids, weights, shared_gate, \
+                     norm_scale)
+  if (dt == TK_F32) {
+    if (sigmoid) ER_LAUNCH(float, true); else ER_LAUNCH(float, false);
+  } else {
+    if (sigmoid) ER_LAUNCH(bf16_t, true); else ER_LAUNCH(bf16_t, false);
+  }
+#undef ER_LAUNCH
   TK_CHECK_LAUNCH("expert_route");
   return 0;
 }
 
 // --------------------------------------------------------------------------
 // inter[pair, j] = silu(W_gate[e] h)_j * (W_up[e] h)_j for pair = (token, place), e = ids[pair] a routed
-// expert (others are skipped).  w_gate_up: [experts][2 * ff][width], gate rows first.
+// expert (others are skipped).  w_gate_up: [experts][2 * ff][width], gate rows first.  `in_weights` (null or a number
+// a pair): the expert reads in_weights[pair] * h; the products being linear, the factor goes on their 32-bit sums.
 // Workgroup (pair, block of EX_ROWS outputs), a wavefront an output at a time.
 // --------------------------------------------------------------------------
 #define EX_ROWS 4  // one output a wavefront: a step of few tokens is a chain of loads, so many short workgroups
 template <typename T>
 __global__ __launch_bounds__(256) void expert_gate_up_kernel(
     const T* __restrict__ h, int h_stride, const T* __restrict__ w_gate_up, const int* __restrict__ ids,
-    T* __restrict__ inter, int width, int ff, int experts, int top) {
+    const float* __restrict__ in_weights, T* __restrict__ inter, int width, int ff, int experts, int top) {
   const int pair = blockIdx.x;
   const int e = ids[pair];
   if (e < 0 || e >= experts) return;
@@ -209,6 +219,10 @@ __global__ __launch_bounds__(256) void expert_gate_up_kernel(
     float g, u;
     wave_dot2<T>(wg + (size_t)j * width, wu + (size_t)j * width, row, width, g, u);
     if (lane == 0) {
+      if (in_weights) {
+        g *= in_weights[pair];
+        u *= in_weights[pair];
+      }
       // gate, up and the activation as the storage type sees them, as the dense feed-forward's epilogue
       const float gr = round_to<T>(g), ur = round_to<T>(u);
       const float a = round_to<T>(gr / (1.0f + expf(-gr)));
@@ -217,7 +231,7 @@ __global__ __launch_bounds__(256) void expert_gate_up_kernel(
   }
 }
 
-TK_API int tk_expert_gate_up(int dt, const void* h, int h_stride, const void* w_gate_up, const int* ids, void* inter,
+TK_API int tk_expert_gate_up(int dt, const void* h, int h_stride, const void* w_gate_up, const int* ids, const float* in_weights, void* inter,
                              int tokens, int width, int ff, int experts, int top, hipStream_t stream) {
   TK_REQUIRE(tokens >= 0 && width > 0 && ff > 0 && experts > 0 && top > 0 && h_stride >= width,
              "expert_gate_up: bad sizes tokens=%d width=%d ff=%d experts=%d top=%d", tokens, width, ff, experts, top);
@@ -227,10 +241,10 @@ TK_API int tk_expert_gate_up(int dt, const void* h, int h_stride, const void* w_
   TK_REQUIRE(grid.y < 65536, "expert_gate_up: an expert of %d rows is too large", ff);
   if (dt == TK_F32)
     hipLaunchKernelGGL(expert_gate_up_kernel<float>, grid, dim3(256), 0, stream, (const float*)h, h_stride,
-                       (const float*)w_gate_up, ids, (float*)inter, width, ff, experts, top);
+                       (const float*)w_gate_up, ids, in_weights, (float*)inter, width, ff, experts, top);
   else
     hipLaunchKernelGGL(expert_gate_up_kernel<bf16_t>, grid, dim3(256), 0, stream, (const bf16_t*)h, h_stride,
-                       (const bf16_t*)w_gate_up, ids, (bf16_t*)inter, width, ff, experts, top);
+                       (const bf16_t*)w_gate_up, ids, in_weights, (bf16_t*)inter, width, ff, experts, top);
   TK_CHECK_LAUNCH("expert_gate_up");
   return 0;
 }
@@ -239,14 +253,15 @@ TK_API int tk_expert_gate_up(int dt, const void* h, int h_stride, const void* w_
 // out[t, c] = sum over the places k of token t, in order, of
 //     weights[t, k] * (W_down[e] inter[t, k])_c       e = ids[t, k] a routed expert
 //     weights[t, k] * h[t, c]                         e an identity expert (e >= experts)
-// plus shared_gate[t] * shared[t, c] when a shared expert's output is given.  out is 32-bit.
+// plus shared_gate[t] * shared[t, c] when a shared expert's output is given.  out is 32-bit.  `unit` != 0: a routed
+// expert's output is added as it is (its weight went on what it read).
 // w_down: [experts][width][ff].  Workgroup (token, block of EX_ROWS columns).
 // --------------------------------------------------------------------------
 template <typename T>
 __global__ __launch_bounds__(256) void expert_combine_kernel(
     const T* __restrict__ h, int h_stride, const T* __restrict__ inter, const T* __restrict__ w_down,
     const int* __restrict__ ids, const float* __restrict__ weights, const float* __restrict__ shared,
-    const float* __restrict__ shared_gate, float* __restrict__ out, int width, int ff, int experts, int top) {
+    const float* __restrict__ shared_gate, float* __restrict__ out, int width, int ff, int experts, int top, int unit) {
   const int t = blockIdx.x;
   const int lane = threadIdx.x & (TK_WAVE - 1), wave = threadIdx.x / TK_WAVE, nwaves = blockDim.x / TK_WAVE;
   const int c0 = blockIdx.y * EX_ROWS;
@@ -255,7 +270,7 @@ __global__ __launch_bounds__(256) void expert_combine_kernel(
     for (int k = 0; k < top; ++k) {
       const int e = ids[(size_t)t * top + k];
       if (e < 0) continue;
-      const float g = weights[(size_t)t * top + k];
+      const float g = unit && e < experts ? 1.f : weights[(size_t)t * top + k];
       float y;
       if (e < experts)
         y = round_to<T>(wave_dot<T>(w_down + ((size_t)e * width + c) * ff, inter + ((size_t)t * top + k) * ff, ff));
@@ -270,7 +285,7 @@ __global__ __launch_bounds__(256) void expert_combine_kernel(
 
 TK_API int tk_expert_combine(int dt, const void* h, int h_stride, const void* inter, const void* w_down, const int* ids,
                              const float* weights, const float* shared, const float* shared_gate, float* out, int tokens,
-                             int width, int ff, int experts, int top, hipStream_t stream) {
+                             int width, int ff, int experts, int top, int unit, hipStream_t stream) {
   TK_REQUIRE(tokens >= 0 && width > 0 && ff > 0 && experts > 0 && top > 0 && h_stride >= width,
              "expert_combine: bad sizes tokens=%d width=%d ff=%d experts=%d top=%d", tokens, width, ff, experts, top);
   TK_REQUIRE(h && inter && w_down && ids && weights && out && (!shared || shared_gate), "expert_combine: a pointer is missing");
@@ -280,11 +295,11 @@ TK_API int tk_expert_combine(int dt, const void* h, int h_stride, const void* in
   if (dt == TK_F32)
     hipLaunchKernelGGL(expert_combine_kernel<float>, grid, dim3(256), 0, stream, (const float*)h, h_stride,
                        (const float*)inter, (const float*)w_down, ids, weights, shared, shared_gate, out, width, ff,
-                       experts, top);
+                       experts, top, unit);
   else
     hipLaunchKernelGGL(expert_combine_kernel<bf16_t>, grid, dim3(256), 0, stream, (const bf16_t*)h, h_stride,
                        (const bf16_t*)inter, (const bf16_t*)w_down, ids, weights, shared, shared_gate, out, width, ff,
-                       experts, top);
+                       experts, top, unit);
   TK_CHECK_LAUNCH("expert_combine");
   return 0;
 }

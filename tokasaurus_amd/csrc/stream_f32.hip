@@ -295,54 +295,68 @@ TK_API int tk_cast_rows(int dt, const float* x, void* out, size_t n, hipStream_t
 
 // --------------------------------------------------------------------------
 // One row a workgroup.  Reads x (32-bit) and the branches a, b (32-bit, either may be null),
-// writes x_out = x + mult * (a + b) (32-bit; may be x itself; null when there is no branch and
-// the stream stays as it is) and, for each of up to two norms, the row
+// writes x_out = x + mult * (a + b) + add (32-bit; may be x itself; null when there is neither a branch nor
+// `add`, one row [hidden] that every row gets, and the stream stays as it is) and, for each of up to two norms, the row
 //     x_out / sqrt(mean(x_out^2) + eps) * (offset + w)
+// or, CENTER (a layer norm without a bias), with m = mean(x_out),
+//     (x_out - m) / sqrt(mean((x_out - m)^2) + eps) * (offset + w)
 // rounded once to T.  `offset` is 1 for weights stored around zero, 0 for plain ones.
 // Norm weights are 32-bit.
 // --------------------------------------------------------------------------
-template <typename T>
+template <typename T, bool CENTER>
 __global__ __launch_bounds__(256) void residual_norm_kernel(
-    const float* __restrict__ x, const float* __restrict__ a, const float* __restrict__ b, float mult,
+    const float* __restrict__ x, const float* __restrict__ a, const float* __restrict__ b, float mult, const float* __restrict__ add,
     float* x_out, const float* __restrict__ w1, const float* __restrict__ w2, float offset, float eps,
     T* __restrict__ h1, T* __restrict__ h2, int hidden) {
   __shared__ float red[16];
   const size_t row = (size_t)blockIdx.x * hidden;
-  float ss = 0.f;
+  const bool changed = a || b || add;
+  float ss = 0.f, sum = 0.f;
   for (int i = threadIdx.x; i < hidden; i += blockDim.x) {
     float v = x[row + i];
     if (a || b) {
       float y = a ? a[row + i] : 0.f;
       if (b) y += b[row + i];
       v = fmaf(mult, y, v);
-      x_out[row + i] = v;
     }
-    ss = fmaf(v, v, ss);
+    if (add) v += add[i];
+    if (changed) x_out[row + i] = v;
+    if (CENTER) sum += v;
+    else ss = fmaf(v, v, ss);
   }
   if (!w1 && !w2) return;
+  const float* src = changed ? x_out : x;  // a thread reads back what it wrote
+  float mean = 0.f;
+  if (CENTER) {
+    mean = block_sum(sum, red) / (float)hidden;
+    for (int i = threadIdx.x; i < hidden; i += blockDim.x) {
+      const float d = src[row + i] - mean;
+      ss = fmaf(d, d, ss);
+    }
+  }
   ss = block_sum(ss, red);
   const float rstd = 1.0f / sqrtf(ss / (float)hidden + eps);
-  const float* src = (a || b) ? x_out : x;  // a thread reads back what it wrote
   for (int i = threadIdx.x; i < hidden; i += blockDim.x) {
-    const float n = src[row + i] * rstd;
+    const float n = (CENTER ? src[row + i] - mean : src[row + i]) * rstd;
     if (w1) h1[row + i] = from_f32<T>(n * (offset + w1[i]));
     if (w2) h2[row + i] = from_f32<T>(n * (offset + w2[i]));
   }
 }
 
-// The same with 16 bytes a load and the new row held in registers between the two passes: for
+// The same with 16 bytes a load and the new row held in registers between the passes: for
 // widths that are multiples of 4 up to 4 * 256 * RN_QUADS (one workgroup of 256 threads a row).
 #define RN_QUADS 8
-template <typename T>
+template <typename T, bool CENTER>
 __global__ __launch_bounds__(256) void residual_norm_vec_kernel(
-    const float* __restrict__ x, const float* __restrict__ a, const float* __restrict__ b, float mult,
+    const float* __restrict__ x, const float* __restrict__ a, const float* __restrict__ b, float mult, const float* __restrict__ add,
     float* x_out, const float* __restrict__ w1, const float* __restrict__ w2, float offset, float eps,
     T* __restrict__ h1, T* __restrict__ h2, int hidden) {
   __shared__ float red[16];
   const size_t row = (size_t)blockIdx.x * hidden;
   const int quads = hidden / 4;
+  const bool changed = a || b || add;
   float4 v[RN_QUADS];
-  float ss = 0.f;
+  float ss = 0.f, sum = 0.f;
 #pragma unroll
   for (int j = 0; j < RN_QUADS; ++j) {
     const int i = threadIdx.x + j * 256;
@@ -356,13 +370,32 @@ __global__ __launch_bounds__(256) void residual_norm_vec_kernel(
         }
         v[j].x = fmaf(mult, y.x, v[j].x); v[j].y = fmaf(mult, y.y, v[j].y);
         v[j].z = fmaf(mult, y.z, v[j].z); v[j].w = fmaf(mult, y.w, v[j].w);
-        ((float4*)(x_out + row))[i] = v[j];
       }
-      ss = fmaf(v[j].x, v[j].x, ss); ss = fmaf(v[j].y, v[j].y, ss);
-      ss = fmaf(v[j].z, v[j].z, ss); ss = fmaf(v[j].w, v[j].w, ss);
+      if (add) {
+        const float4 z = ((const float4*)add)[i];
+        v[j].x += z.x; v[j].y += z.y; v[j].z += z.z; v[j].w += z.w;
+      }
+      if (changed) ((float4*)(x_out + row))[i] = v[j];
+      if (CENTER) {
+        sum += (v[j].x + v[j].y) + (v[j].z + v[j].w);
+      } else {
+        ss = fmaf(v[j].x, v[j].x, ss); ss = fmaf(v[j].y, v[j].y, ss);
+        ss = fmaf(v[j].z, v[j].z, ss); ss = fmaf(v[j].w, v[j].w, ss);
+      }
     }
   }
   if (!w1 && !w2) return;
+  if (CENTER) {
+    const float mean = block_sum(sum, red) / (float)hidden;
+#pragma unroll
+    for (int j = 0; j < RN_QUADS; ++j) {
+      if (threadIdx.x + j * 256 < quads) {
+        v[j].x -= mean; v[j].y -= mean; v[j].z -= mean; v[j].w -= mean;
+        ss = fmaf(v[j].x, v[j].x, ss); ss = fmaf(v[j].y, v[j].y, ss);
+        ss = fmaf(v[j].z, v[j].z, ss); ss = fmaf(v[j].w, v[j].w, ss);
+      }
+    }
+  }
   ss = block_sum(ss, red);
   const float rstd = 1.0f / sqrtf(ss / (float)hidden + eps);
 #pragma unroll
@@ -386,30 +419,26 @@ __global__ __launch_bounds__(256) void residual_norm_vec_kernel(
   }
 }
 
-TK_API int tk_residual_norm(int dt, const float* x, const float* a, const float* b, float mult,
-                            float* x_out, const float* w1, const float* w2, float offset, float eps,
+TK_API int tk_residual_norm(int dt, const float* x, const float* a, const float* b, float mult, const float* add,
+                            float* x_out, const float* w1, const float* w2, float offset, float eps, int center,
                             void* h1, void* h2, int rows, int hidden, hipStream_t stream) {
   TK_REQUIRE(rows >= 0 && hidden > 0, "residual_norm: bad sizes %d %d", rows, hidden);
-  TK_REQUIRE(!(a || b) || x_out, "residual_norm: a branch needs a place for the new stream");
+  TK_REQUIRE(!(a || b || add) || x_out, "residual_norm: a branch needs a place for the new stream");
   TK_REQUIRE((!w1 || h1) && (!w2 || h2), "residual_norm: a norm needs a place for its rows");
   if (rows == 0) return 0;
-  const uintptr_t all = (uintptr_t)x | (uintptr_t)a | (uintptr_t)b | (uintptr_t)x_out | (uintptr_t)w1 | (uintptr_t)w2;
-  if (hidden % 4 == 0 && hidden <= 4 * 256 * RN_QUADS && (all & 15) == 0) {
-    if (dt == TK_F32)
-      hipLaunchKernelGGL(residual_norm_vec_kernel<float>, dim3(rows), dim3(256), 0, stream, x, a, b, mult, x_out, w1, w2,
-                         offset, eps, (float*)h1, (float*)h2, hidden);
-    else
-      hipLaunchKernelGGL(residual_norm_vec_kernel<bf16_t>, dim3(rows), dim3(256), 0, stream, x, a, b, mult, x_out, w1, w2,
-                         offset, eps, (bf16_t*)h1, (bf16_t*)h2, hidden);
-    TK_CHECK_LAUNCH("residual_norm");
-    return 0;
-  }
-  if (dt == TK_F32)
-    hipLaunchKernelGGL(residual_norm_kernel<float>, dim3(rows), dim3(256), 0, stream, x, a, b, mult,
-                       x_out, w1, w2, offset, eps, (float*)h1, (float*)h2, hidden);
-  else
-    hipLaunchKernelGGL(residual_norm_kernel<bf16_t>, dim3(rows), dim3(256), 0, stream, x, a, b, mult,
-                       x_out, w1, w2, offset, eps, (bf16_t*)h1, (bf16_t*)h2, hidden);
+  const uintptr_t all = (uintptr_t)x | (uintptr_t)a | (uintptr_t)b | (uintptr_t)add | (uintptr_t)x_out | (uintptr_t)w1 | (uintptr_t)w2;
+  const bool vec = hidden % 4 == 0 && hidden <= 4 * 256 * RN_QUADS && (all & 15) == 0;
+#define RN_LAUNCH(K, T, C)                                                                                                     \
+  hipLaunchKernelGGL((K<T, C>), dim3(rows), dim3(256), 0, stream, x, a, b, mult, add, x_out, w1, w2, offset, eps, (T*)h1, (T*)h2, hidden)
+#define RN_CASE(K)                                                                    \
+  do {                                                                                \
+    if (dt == TK_F32) { if (center) RN_LAUNCH(K, float, true); else RN_LAUNCH(K, float, false); } \
+    else { if (center) RN_LAUNCH(K, bf16_t, true); else RN_LAUNCH(K, bf16_t, false); }  \
+  } while (0)
+  if (vec) RN_CASE(residual_norm_vec_kernel);
+  else RN_CASE(residual_norm_kernel);
+#undef RN_CASE
+#undef RN_LAUNCH
   TK_CHECK_LAUNCH("residual_norm");
   return 0;
 }

@@ -46,9 +46,13 @@ _SIGNATURES: dict[str, dict[str, list]] = {
         "tk_sigmoid_gate": [c_int, _P, c_int, _P, c_int, c_float, _P, c_int, c_int, c_int, _P],
         "tk_short_conv": [c_int, _P, c_int, _P, c_int, _P, c_size_t, _P, _P, _P, _P] + [c_int] * 4 + [_P],
         "tk_gelu_glu": [c_int, _P, _P, c_int, c_int, _P],
-        "tk_residual_norm": [c_int, _P, _P, _P, c_float, _P, _P, _P, c_float, c_float, _P, _P, c_int, c_int, _P],
+        "tk_residual_norm": [c_int, _P, _P, _P, c_float, _P, _P, _P, _P, c_float, c_float, c_int, _P, _P, c_int, c_int, _P],
+        "tk_state_space": [_P, c_int, c_int, c_int, _P, _P, c_int, _P, _P, _P, _P, c_size_t, c_size_t, _P, _P, _P, _P, _P, _P] + [c_int] * 7 + [_P],
+        "tk_state_space_rec_width": [c_int] * 4,
+        "tk_gate_group_norm": [c_int, _P, _P, c_int, _P, c_float, _P, c_int, c_int, c_int, _P],
+        "tk_rotate_heads": [c_int, _P, c_int, _P, _P] + [c_int] * 5 + [c_float, _P],
         "tk_softcap": [_P, c_size_t, c_float, _P],
-        "tk_qk_prepare": [c_int, _P, c_int, _P, _P, _P, c_int, _P, _P, c_float, _P, _P, _P] + [c_int] * 13 + [_P, c_int, c_float, _P],
+        "tk_qk_prepare": [c_int, _P, c_int, _P, _P, _P, c_int, _P, _P, c_float, _P, _P, _P] + [c_int] * 13 + [_P, c_int, c_float, c_int, _P],
         "tk_unrotate_gate": [c_int, _P, c_int, _P, _P, c_int, _P, c_int, c_int, c_int, c_int, _P],
         "tk_min_gru": [c_int, _P, c_int, _P, _P, c_size_t, _P, _P, _P, c_int, c_int, c_int, _P],
         "tk_embed_bigram": [c_int, _P, _P, _P, _P, _P, _P, _P, _P, _P, _P, _P, c_int, c_int, c_int, c_float, c_int, c_int, c_int, _P],
@@ -58,9 +62,9 @@ _SIGNATURES: dict[str, dict[str, list]] = {
         "tk_gather_keys": [c_int, _P, _P, c_int, _P, _P, _P] + [c_int] * 5 + [_P],
         "tk_post_norm_residual": [c_int, _P, _P, _P, c_float, _P, _P, c_float, _P, c_int, c_int, _P],
         "tk_concat_cast": [c_int, _P, _P, _P, c_int, c_int, _P],
-        "tk_expert_route": [c_int, _P, c_int, _P, _P, _P] + [c_int] * 6 + [_P, _P, _P, c_float, _P],
-        "tk_expert_gate_up": [c_int, _P, c_int, _P, _P, _P] + [c_int] * 5 + [_P],
-        "tk_expert_combine": [c_int, _P, c_int, _P, _P, _P, _P, _P, _P, _P] + [c_int] * 5 + [_P],
+        "tk_expert_route": [c_int, _P, c_int, _P, _P, _P] + [c_int] * 6 + [_P, _P, _P, c_float, c_int, _P],
+        "tk_expert_gate_up": [c_int, _P, c_int, _P, _P, _P, _P] + [c_int] * 5 + [_P],
+        "tk_expert_combine": [c_int, _P, c_int, _P, _P, _P, _P, _P, _P, _P] + [c_int] * 6 + [_P],
         "tk_head_linear": [c_int, _P, c_int, _P, _P, c_int, c_int] + [c_int] * 4 + [_P],
         "tk_squared_relu": [c_int, _P, c_size_t, _P],
         "tk_attention_tile_f32": [c_int, _P, c_int, _P, c_int, _P, _P, _P, c_int, _P, _P, _P, _P] + [c_int] * 7
@@ -86,9 +90,9 @@ _SIGNATURES: dict[str, dict[str, list]] = {
         "tk_gemm_skinny_bf16": [_P, c_int, _P, _P, c_int, _P, c_int, _P] + [c_int] * 9 + [_P],
         "tk_gemm_skinny_parts": [c_int, c_int, c_int],
         "tk_grouped_gemm_bf16": [_P, c_int, _P, _P, _P, c_int, c_int, c_int, c_int, _P, c_size_t, _P, c_int, c_int, c_int, c_int,
-                                 c_int, c_int, _P],
+                                 c_int, c_int, _P, _P, _P],
         "tk_expert_sort": [_P, c_int, c_int, c_int, c_int, _P, _P, _P, _P],
-        "tk_expert_sum": [_P, c_int, _P, _P, _P, _P, _P, _P, c_int, c_int, c_int, c_int, _P],
+        "tk_expert_sum": [_P, c_int, _P, _P, _P, _P, _P, _P, c_int, c_int, c_int, c_int, c_int, _P],
     },
     "library": {
         "tk_gemm_library_bf16": [_P, c_int, _P, c_int, _P, c_int, c_int, c_int, c_int, c_int, _P, c_size_t, _P],

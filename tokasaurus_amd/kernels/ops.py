@@ -1343,6 +1343,73 @@ def short_conv(h: torch.Tensor, weight: torch.Tensor, tails: torch.Tensor | None
     return out
 
 
+def state_space_sizes(heads: int, groups: int, state: int, value_dim: int, taps: int) -> tuple[int, int]:
+    """32-bit numbers a request keeps for one ``state_space`` mixer, and the place among them where the ring of the
+    convolution's last inputs begins: the matrices [heads][value_dim][state], then [taps][channels]."""
+    ring = -(-heads * value_dim * state // 4) * 4
+    channels = heads * value_dim + 2 * groups * state
+    return -(-(ring + (taps * channels if taps > 1 else 0)) // 4) * 4, ring
+
+
+def state_space(proj: torch.Tensor, x_off: int, dt_off: int, conv_w: torch.Tensor, conv_b: torch.Tensor, a_log: torch.Tensor,
+                dt_bias: torch.Tensor, d_skip: torch.Tensor, state: torch.Tensor, q_start: torch.Tensor, token_req: torch.Tensor,
+                slots: torch.Tensor, positions: torch.Tensor, heads: int, groups: int, state_dim: int, value_dim: int,
+                longest: int | None = None) -> torch.Tensor:
+    """A selective state-space recurrence over every request's tokens of this step, from the 32-bit sums ``proj`` of one
+    stacked product: columns x | B | C (heads * value_dim, groups * state_dim, groups * state_dim) from ``x_off`` on pass
+    a causal convolution per channel (``conv_w`` [taps, channels] tap by tap, the last the current token's; ``conv_b``)
+    and silu; dt = softplus(columns from ``dt_off`` on + ``dt_bias``), one a head; per head with the B and C of its group
+    ``S <- exp(-exp(a_log) dt) S + dt B x^T``, ``y = S^T C + d_skip x``.  ``state`` [slots + 1, ``state_space_sizes``]
+    (32-bit) is read and written in the requests' ``slots``.  ``longest``: the most tokens a request brings in this step
+    (the launch's form depends on it, the sums do not).  Returns y [tokens, heads * value_dim] in 32-bit."""
+    _gpu(proj, conv_w, conv_b, a_log, dt_bias, d_skip, state, q_start, token_req, slots, positions)
+    H, G, N, dv = int(heads), int(groups), int(state_dim), int(value_dim)
+    _need(proj.dim() == 2 and proj.dtype == torch.float32 and proj.stride(1) == 1, "state_space: 32-bit rows with unit inner stride")
+    n, width = proj.shape
+    channels = H * dv + 2 * G * N
+    _need(0 <= x_off and x_off + channels <= width and 0 <= dt_off and dt_off + H <= width, "state_space: a part lies outside the rows")
+    _need(conv_w.dim() == 2 and conv_w.shape[1] == channels and conv_w.dtype == torch.float32 and conv_w.is_contiguous(),
+          "state_space: taps must be contiguous float32 [taps, channels]")
+    taps = conv_w.shape[0]
+    _f32_vector(conv_b, channels, "state_space: the convolution's bias")
+    for v, name in ((a_log, "the decays' logarithms"), (dt_bias, "the step sizes' bias"), (d_skip, "the skip's factors")):
+        _f32_vector(v, H, f"state_space: {name}")
+    size, ring = state_space_sizes(H, G, N, dv, taps)
+    _need(state.dim() == 2 and state.dtype == torch.float32 and state.is_contiguous() and state.shape[1] >= size,
+          "state_space: the state must be contiguous float32 rows of state_space_sizes")
+    for t, name in ((q_start, "q_start"), (token_req, "token_req"), (slots, "slots"), (positions, "positions")):
+        _i32(t, name)
+    _need(token_req.numel() == n and positions.numel() == n and q_start.numel() == slots.numel() + 1,
+          "state_space: one request and one position a token, one slot a request")
+    _need(N <= 512, f"state_space: heads of up to 512 rows of state, not {N}")
+    y = torch.empty((n, H * dv), dtype=torch.float32, device=proj.device)
+    if n:
+        longest = max(1, int(n if longest is None else longest))
+        rec = (torch.empty((n, load("core").tk_state_space_rec_width(H, G, N, dv)), dtype=torch.float32, device=proj.device)
+               if longest > 1 else None)
+        call("tk_state_space", proj.data_ptr(), proj.stride(0), int(x_off), int(dt_off), conv_w.data_ptr(), conv_b.data_ptr(), taps,
+             a_log.data_ptr(), dt_bias.data_ptr(), d_skip.data_ptr(), state.data_ptr(), state.stride(0), ring, q_start.data_ptr(),
+             token_req.data_ptr(), slots.data_ptr(), positions.data_ptr(), rec.data_ptr() if rec is not None else None, y.data_ptr(), n,
+             slots.numel(), H, G, N, dv, longest, _stream())
+    return y
+
+
+def gate_group_norm(y: torch.Tensor, z: torch.Tensor, weight: torch.Tensor, eps: float, groups: int, out_dtype: torch.dtype) -> torch.Tensor:
+    """v = y * silu(z) (32-bit rows; ``z`` a 2-d view, rows a stride apart), every one of ``groups`` equal parts of a row of
+    v divided by its root mean square, times ``weight`` (32-bit, the whole row's size); rounded once to ``out_dtype``."""
+    _gpu(y, z, weight)
+    _need(y.dim() == 2 and y.dtype == torch.float32 and y.is_contiguous() and y.shape[1] % groups == 0,
+          "gate_group_norm: contiguous float32 rows of equal parts")
+    _need(z.shape == y.shape and z.dtype == torch.float32 and z.stride(1) == 1, "gate_group_norm: a 32-bit gate of the rows' shape")
+    n, width = y.shape
+    _f32_vector(weight, width, "gate_group_norm: the weight")
+    out = torch.empty((n, width), dtype=out_dtype, device=y.device)
+    if n:
+        call("tk_gate_group_norm", dtype_code(out_dtype), y.data_ptr(), z.data_ptr(), z.stride(0), weight.data_ptr(), float(eps),
+             out.data_ptr(), n, int(groups), width // int(groups), _stream())
+    return out
+
+
 def gelu_glu(gate_up: torch.Tensor) -> torch.Tensor:
     """[rows, 2I] laid out [gate | up] -> gelu(gate) * up with the tanh form of gelu, [rows, I]; 32-bit arithmetic, one rounding."""
     _gpu(gate_up)
@@ -1364,16 +1431,20 @@ def residual_norm(
     eps: float = 0.0,
     out_dtype: torch.dtype = torch.float32,
     in_place: bool = True,
+    add_row: torch.Tensor | None = None,
+    center: bool = False,
 ) -> tuple[torch.Tensor, torch.Tensor | None, torch.Tensor | None]:
     """The update of a 32-bit residual stream and the norms that read the new stream, in one pass:
     ``x_new = x + mult * (a + b)`` for the 32-bit ``branches`` (either may be None; with neither
     the stream stays), then for each of up to two 32-bit ``weights`` the rows
     ``x_new / sqrt(mean(x_new^2) + eps) * (w + (1 if unit_offset else 0))`` rounded once to
     ``out_dtype``.  Returns (x_new, normed rows for weights[0], for weights[1]).  ``in_place``:
-    the new stream overwrites ``x``."""
+    the new stream overwrites ``x``.  ``add_row`` (32-bit [H]): one row that is added to every row of the
+    stream, after the branches.  ``center``: layer norms without a bias, i.e. the rows' means are taken off first."""
     a, b = branches
     w1, w2 = weights
-    _gpu(x, a, b, w1, w2)
+    _gpu(x, a, b, w1, w2, add_row)
+    _f32_vector(add_row, x.shape[-1], "residual_norm: the added row")
     _need(x.dim() == 2 and x.dtype == torch.float32 and x.is_contiguous(), "residual_norm: the stream must be contiguous float32 [rows, H]")
     rows, hidden = x.shape
     for y in (a, b):
@@ -1381,16 +1452,16 @@ def residual_norm(
               "residual_norm: a branch must be contiguous float32 of the stream's shape")
     _f32_vector(w1, hidden, "residual_norm: a norm weight")
     _f32_vector(w2, hidden, "residual_norm: a norm weight")
-    changed = a is not None or b is not None
+    changed = a is not None or b is not None or add_row is not None
     x_out = (x if in_place else torch.empty_like(x)) if changed else x
     h1 = torch.empty((rows, hidden), dtype=out_dtype, device=x.device) if w1 is not None else None
     h2 = torch.empty((rows, hidden), dtype=out_dtype, device=x.device) if w2 is not None else None
     if rows == 0:
         return x_out, h1, h2
     call("tk_residual_norm", dtype_code(out_dtype), x.data_ptr(), a.data_ptr() if a is not None else None,
-         b.data_ptr() if b is not None else None, float(mult), x_out.data_ptr() if changed else None,
-         w1.data_ptr() if w1 is not None else None, w2.data_ptr() if w2 is not None else None,
-         1.0 if unit_offset else 0.0, float(eps), h1.data_ptr() if h1 is not None else None,
+         b.data_ptr() if b is not None else None, float(mult), add_row.data_ptr() if add_row is not None else None,
+         x_out.data_ptr() if changed else None, w1.data_ptr() if w1 is not None else None, w2.data_ptr() if w2 is not None else None,
+         1.0 if unit_offset else 0.0, float(eps), 1 if center else 0, h1.data_ptr() if h1 is not None else None,
          h2.data_ptr() if h2 is not None else None, rows, hidden, _stream())
     return x_out, h1, h2
 
@@ -1534,6 +1605,7 @@ def qk_prepare(
     value_freq: torch.Tensor | None = None,
     value_pair_halves: bool = False,
     rotation_scale: float = 1.0,
+    rotate_queries: bool = True,
 ) -> None:
     """In place on the rows [q: nq*dq | k: nkv*dk | v: nkv*dv] (only q when not ``write_cache``):
     the RMS norm of the whole query row and of the whole key row (32-bit weights of those sizes,
@@ -1565,7 +1637,7 @@ def qk_prepare(
     _f32_vector(value_freq, value_dim // 2, "qk_prepare: the values' frequencies")
     rot = 0
     if freq is not None:
-        _need(freq.dim() == 1 and freq.dtype == torch.float32 and freq.is_contiguous() and 2 * freq.numel() <= min(key_dim, dq),
+        _need(freq.dim() == 1 and freq.dtype == torch.float32 and freq.is_contiguous() and 2 * freq.numel() <= (min(key_dim, dq) if rotate_queries else key_dim),
               "qk_prepare: frequencies must be contiguous float32, at most half a head's size of them")
         rot = 2 * freq.numel()
     if write_cache:
@@ -1580,7 +1652,22 @@ def qk_prepare(
          n, nq, nkv if write_cache else 0, dq, key_dim, value_dim, rot, page_size, 1 if write_cache else 0,
          1 if pair_halves else 0, 1 if values_are_keys else 0, 1 if per_head else 0, key_skip,
          value_freq.data_ptr() if value_freq is not None else None, 1 if value_pair_halves else 0, float(rotation_scale),
-         _stream())
+         1 if rotate_queries else 0, _stream())
+
+
+def rotate_heads_(x: torch.Tensor, positions: torch.Tensor, freq: torch.Tensor, heads: int, head_dim: int, pair_halves: bool,
+                  rotation_scale: float = 1.0) -> torch.Tensor:
+    """In place on the rows [heads * head_dim]: the leading 2 * len(freq) elements of every head turned by position *
+    freq[i], pairs (i, i + len(freq)) with ``pair_halves`` and (2i, 2i + 1) without; cosines and sines times ``rotation_scale``."""
+    _gpu(x, positions, freq)
+    _need(x.dim() == 2 and x.stride(1) == 1 and x.shape[1] >= heads * head_dim, "rotate_heads: rows of unit inner stride that hold the heads")
+    _i32(positions, "positions")
+    _need(positions.numel() == x.shape[0], "rotate_heads: one position a row")
+    _need(freq.dim() == 1 and freq.dtype == torch.float32 and freq.is_contiguous() and 0 < 2 * freq.numel() <= head_dim,
+          "rotate_heads: frequencies must be contiguous float32, at most half a head's size of them")
+    call("tk_rotate_heads", dtype_code(x.dtype), x.data_ptr(), x.stride(0), positions.data_ptr(), freq.data_ptr(), x.shape[0], int(heads),
+         int(head_dim), 2 * freq.numel(), 1 if pair_halves else 0, float(rotation_scale), _stream())
+    return x
 
 
 def gather_keys(kcache: torch.Tensor, block_table: torch.Tensor, req: torch.Tensor, pos: torch.Tensor, key_dim: int,
@@ -1888,7 +1975,7 @@ def head_linear(x: torch.Tensor, w: torch.Tensor, out_f32: bool = False) -> torc
         # many rows: tiles of 32 rows on the matrix cores, the head as the tile's group
         tiles = -(-x.shape[0] // GROUPED_TILE)
         call("tk_grouped_gemm_bf16", x.data_ptr(), x.stride(0), None, None, None, tiles, heads, n_in, n_out, w.data_ptr(),
-             n_out * n_in, y.data_ptr(), y.stride(0), n_out, n_in, x.shape[0], 0, 1 if out_f32 else 0, _stream())
+             n_out * n_in, y.data_ptr(), y.stride(0), n_out, n_in, x.shape[0], 0, 1 if out_f32 else 0, None, None, _stream())
         return y
     if x.shape[0]:
         call("tk_head_linear", dtype_code(x.dtype), x.data_ptr(), x.stride(0), w.data_ptr(), y.data_ptr(), y.stride(0),
@@ -1896,11 +1983,11 @@ def head_linear(x: torch.Tensor, w: torch.Tensor, out_f32: bool = False) -> torc
     return y
 
 
-def expert_route(h: torch.Tensor, w_router: torch.Tensor, correction: torch.Tensor, groups: int, keep: int, top: int,
+def expert_route(h: torch.Tensor, w_router: torch.Tensor, correction: torch.Tensor | None, groups: int, keep: int, top: int,
                  w_gate: torch.Tensor | None = None, normalize_scale: float | None = None,
-                 unit_gate: bool = False) -> tuple[torch.Tensor, torch.Tensor, torch.Tensor | None]:
+                 unit_gate: bool = False, sigmoid_scores: bool = False) -> tuple[torch.Tensor, torch.Tensor, torch.Tensor | None]:
     """The router of a mixture of experts, 32-bit arithmetic: logits ``w_router h`` over all
-    experts, their softmax s, the choice by ``s + correction`` among the experts of the ``keep``
+    experts, their softmax s (or, ``sigmoid_scores``, the sigmoid of each), the choice by ``s + correction`` (None: by s) among the experts of the ``keep``
     groups of neighbours (of ``groups`` equal ones) whose best choice score is largest, ties to the
     left.  Returns ids [tokens, top] int32 in the order of the choice scores, weights [tokens, top]
     (the chosen experts' s), and, with ``w_gate`` [width], sigmoid(w_gate . h) [tokens].  ``normalize_scale``: the
@@ -1919,19 +2006,23 @@ def expert_route(h: torch.Tensor, w_router: torch.Tensor, correction: torch.Tens
     gate = torch.empty((n,), dtype=torch.float32, device=h.device) if (w_gate is not None or unit_gate) else None
     if n == 0:
         return ids, weights, gate
-    call("tk_expert_route", dtype_code(h.dtype), h.data_ptr(), h.stride(0), w_router.data_ptr(), correction.data_ptr(),
-         w_gate.data_ptr() if w_gate is not None else None, n, width, n_all, int(groups), int(keep), int(top),
+    call("tk_expert_route", dtype_code(h.dtype), h.data_ptr(), h.stride(0), w_router.data_ptr(),
+         correction.data_ptr() if correction is not None else None, w_gate.data_ptr() if w_gate is not None else None, n, width, n_all, int(groups), int(keep), int(top),
          ids.data_ptr(), weights.data_ptr(), gate.data_ptr() if gate is not None else None,
-         float(normalize_scale) if normalize_scale else 0.0, _stream())
+         float(normalize_scale) if normalize_scale else 0.0, 1 if sigmoid_scores else 0, _stream())
     return ids, weights, gate
 
 
 def expert_mix(h: torch.Tensor, w_gate_up: torch.Tensor, w_down: torch.Tensor, ids: torch.Tensor, weights: torch.Tensor,
-               shared: torch.Tensor | None = None, shared_gate: torch.Tensor | None = None) -> torch.Tensor:
+               shared: torch.Tensor | None = None, shared_gate: torch.Tensor | None = None,
+               weights_on_input: bool = False) -> torch.Tensor:
     """The weighted sum of a token's chosen experts, 32-bit [tokens, width]: expert e is
     ``w_down[e] (silu(gate) * up)`` with [gate | up] = ``w_gate_up[e] h``; an id from
     ``len(w_down)`` on names an identity expert (its output is h), a negative id an empty
-    place.  ``shared`` (32-bit [tokens, width]) times ``shared_gate`` [tokens] is added."""
+    place.  ``shared`` (32-bit [tokens, width]) times ``shared_gate`` [tokens] is added.  ``weights_on_input``: a chosen
+    expert reads weight * h and its output is added as it is (the factor goes on the 32-bit sums of gate and up)."""
+    unit = 1 if weights_on_input else 0
+    on_input = weights.data_ptr() if weights_on_input else None
     _gpu(h, w_gate_up, w_down, ids, weights, shared, shared_gate)
     experts, two_ff, width = w_gate_up.shape
     ff = two_ff // 2
@@ -1959,18 +2050,19 @@ def expert_mix(h: torch.Tensor, w_gate_up: torch.Tensor, w_down: torch.Tensor, i
              tile_group.data_ptr(), _stream())
         inter = torch.empty((slots, ff), dtype=h.dtype, device=h.device)
         call("tk_grouped_gemm_bf16", h.data_ptr(), h.stride(0), slot_token.data_ptr(), None, tile_group.data_ptr(), max_tiles, 0,
-             0, 0, w_gate_up.data_ptr(), 2 * ff * width, inter.data_ptr(), ff, ff, width, slots, 1, 0, _stream())
+             0, 0, w_gate_up.data_ptr(), 2 * ff * width, inter.data_ptr(), ff, ff, width, slots, 1, 0, on_input,
+             slot_pair.data_ptr() if weights_on_input else None, _stream())
         y = torch.empty((n * top, width), dtype=h.dtype, device=h.device)
         call("tk_grouped_gemm_bf16", inter.data_ptr(), ff, None, slot_pair.data_ptr(), tile_group.data_ptr(), max_tiles, 0,
-             0, 0, w_down.data_ptr(), width * ff, y.data_ptr(), width, width, ff, slots, 0, 0, _stream())
+             0, 0, w_down.data_ptr(), width * ff, y.data_ptr(), width, width, ff, slots, 0, 0, None, None, _stream())
         call("tk_expert_sum", h.data_ptr(), h.stride(0), y.data_ptr(), ids.data_ptr(), weights.data_ptr(),
              shared.data_ptr() if shared is not None else None, shared_gate.data_ptr() if shared is not None else None,
-             out.data_ptr(), n, width, experts, top, _stream())
+             out.data_ptr(), n, width, experts, top, unit, _stream())
         return out
     inter = torch.empty((n * top, ff), dtype=h.dtype, device=h.device)
-    call("tk_expert_gate_up", dtype_code(h.dtype), h.data_ptr(), h.stride(0), w_gate_up.data_ptr(), ids.data_ptr(),
+    call("tk_expert_gate_up", dtype_code(h.dtype), h.data_ptr(), h.stride(0), w_gate_up.data_ptr(), ids.data_ptr(), on_input,
          inter.data_ptr(), n, width, ff, experts, top, _stream())
     call("tk_expert_combine", dtype_code(h.dtype), h.data_ptr(), h.stride(0), inter.data_ptr(), w_down.data_ptr(),
          ids.data_ptr(), weights.data_ptr(), shared.data_ptr() if shared is not None else None,
-         shared_gate.data_ptr() if shared is not None else None, out.data_ptr(), n, width, ff, experts, top, _stream())
+         shared_gate.data_ptr() if shared is not None else None, out.data_ptr(), n, width, ff, experts, top, unit, _stream())
     return out

@@ -10,7 +10,7 @@ from tokasaurus_amd.kernels import ops
 from tokasaurus_amd.models.spec import ModelSpec
 from tokasaurus_amd.parts.base import (BLOCKS, CONNECTORS, EMBEDDINGS, HEADS, CacheNeed, CacheView, Part, Prepared, StateNeed, StepContext,
                                        TensorSpec)
-from tokasaurus_amd.parts.block import build_with_shared, stream_and_prepared
+from tokasaurus_amd.parts.block import PendingSum, build_with_shared, stream_and_prepared
 import tokasaurus_amd.parts.embedding  # noqa: F401  (registers the embedding and the head)
 from tokasaurus_amd.parts.linear import Placer
 
@@ -88,7 +88,7 @@ class CausalLM:
         order = self.spec.run_order
         last = len(order) - 1
         # a connector reads the embedding's output again; blocks may update the stream in place
-        x0 = x.clone() if any(not getattr(c, "takes_history", False) for c in self.connectors) else None
+        x0 = (x.clone() if any(not getattr(c, "takes_history", False) and not c.updates_stream for c in self.connectors) else None)
         # connectors that read every stream so far: the embedding's output and each block's result are kept side by
         # side, [streams, tokens, H]; a block updates its input in place, so its input is a copy in the next place
         hist = None
@@ -99,10 +99,15 @@ class CausalLM:
             hist[0].copy_(x)
             hist[1].copy_(x)
             x = hist[1]
+        tap = ctx.extras.get("model_tap")  # a list that collects the stream every run entry leaves (tests, debugging)
+        handed: PendingSum | None = None  # the branch that the block in front has left to the connector before this entry
         for i, entry in enumerate(order):
             rows = want_rows if i == last else None
             block = self.blocks[entry.layer]
-            if entry.before is not None:
+            if entry.before is not None and self.connectors[entry.before].updates_stream:
+                out = self.connectors[entry.before].update(x, handed, block.entry_norm() if block.fuses_norm else None)
+                (x, prepared), handed = stream_and_prepared(out), None
+            elif entry.before is not None:
                 x, prepared = self.connectors[entry.before].forward(x, x0), None
                 if hist is not None:
                     hist[i + 1].copy_(x)
@@ -118,6 +123,11 @@ class CausalLM:
                 # the block hands its branches over unsummed: the connector behind it adds them in its own pass
                 pending = block.forward(x, ctx, caches[i], states[i], rows, prepared=prepared, next_norm=None, defer_sum=True)
                 out = pending.x
+            elif (i < last and tap is None and hist is None and after is None and order[i + 1].before is not None
+                  and self.connectors[order[i + 1].before].updates_stream and getattr(block, "can_defer_sum", False)):
+                # the block hands its last branch over unsummed: the connector before the next block adds it in its own pass
+                handed = block.forward(x, ctx, caches[i], states[i], rows, prepared=prepared, next_norm=None, defer_sum=True)
+                out = handed.x
             elif block.fuses_norm:
                 # (a connector behind this block changes the stream before anything reads it)
                 out = block.forward(x, ctx, caches[i], states[i], rows, prepared=prepared,
@@ -139,8 +149,7 @@ class CausalLM:
                     x = hist[i + 2]
             elif entry.after is not None:
                 raise RuntimeError("a connector behind a run entry reads the model's streams so far (takes_history)")
-            tap = ctx.extras.get("model_tap")
-            if tap is not None:  # a list that collects the stream every run entry leaves (tests, debugging)
+            if tap is not None:
                 tap.append(x.clone())
         if last < 0 and want_rows is not None:
             x = ops.gather_rows(x, want_rows)

@@ -20,6 +20,8 @@ from tokasaurus_amd.config.sakevik_config import SakevikConfig
 from tokasaurus_amd.models.sakevik import sakevik_spec
 from tokasaurus_amd.config.sazilorn_config import SazilornConfig
 from tokasaurus_amd.models.sazilorn import sazilorn_spec
+from tokasaurus_amd.config.vekasun_config import VekasunConfig
+from tokasaurus_amd.models.vekasun import vekasun_spec
 from tokasaurus_amd.models.spec import ModelSpec
 
 
@@ -47,6 +49,7 @@ register_architecture(Architecture("kupuzen", KupuzenConfig.from_dict, kupuzen_s
 register_architecture(Architecture("taborax", TaboraxConfig.from_dict, taborax_spec, class_names=("Taborax",)))
 register_architecture(Architecture("sakevik", SakevikConfig.from_dict, sakevik_spec, class_names=("Sakevik",)))
 register_architecture(Architecture("sazilorn", SazilornConfig.from_dict, sazilorn_spec, class_names=("Sazilorn",)))
+register_architecture(Architecture("vekasun", VekasunConfig.from_dict, vekasun_spec, class_names=("Vekasun",)))
 
 
 def architecture_of(config_dict: dict[str, Any]) -> Architecture:

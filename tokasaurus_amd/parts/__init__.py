@@ -2,7 +2,7 @@
 built-in parts under their names."""
 
 from tokasaurus_amd.parts import (attention, block, delta_rule, embedding, feedforward, grouped_attention, latent_attention, linear_attention, min_gru, mixer_pair,  # noqa: F401
-                                   norm, position, routed_experts)
+                                   norm, position, routed_experts, state_space)
 from tokasaurus_amd.parts.base import (  # noqa: F401
     BLOCKS,
     EMBEDDINGS,

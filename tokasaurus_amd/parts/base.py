@@ -294,7 +294,12 @@ class Connector(Part):
     """What a model does to its residual stream between two blocks, outside any block: it gets
     the stream ``x`` and the embedding's output ``x0`` of the same rows and returns the new
     stream (a new tensor: ``x0`` is read again later).  A run entry names the connector that
-    runs before it (``models.spec.RunEntry.before``)."""
+    runs before it (``models.spec.RunEntry.before``).  A connector that reads the stream alone says
+    ``updates_stream = True`` and has ``update(x, pending, next_norm)`` instead: it changes ``x`` in place, adds
+    the branch that the block in front has handed over unsummed (``parts.block.PendingSum`` or None) in the same pass,
+    and may return (stream, ``Prepared``) for the norm that reads it."""
+
+    updates_stream = False
 
     def forward(self, x: torch.Tensor, x0: torch.Tensor) -> torch.Tensor:
         raise NotImplementedError

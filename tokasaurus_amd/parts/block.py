@@ -29,7 +29,7 @@ from tokasaurus_amd.parts.base import (
     StepContext,
     TensorSpec,
 )
-from tokasaurus_amd.parts.base import AVERAGE_WEIGHT
+from tokasaurus_amd.parts.base import AVERAGE_WEIGHT, MATRIX
 from tokasaurus_amd.parts.linear import Linear, Placer
 from tokasaurus_amd.parts.short_conv import ShortConvResidual
 
@@ -370,6 +370,101 @@ class PostNormBlock(Block):
         if h is None or reader is None:
             return x
         return x, Prepared(None, reader, h)
+
+
+def _update_stream(x: torch.Tensor, branches: tuple, reader, mult: float = 1.0, add_row: torch.Tensor | None = None):
+    """x <- x + mult * (branches) + add_row on a 32-bit stream, in place, with the rows of the norm that reads it where
+    that norm can be written in the same pass (it has ``update``): (stream, ``Prepared`` or None)."""
+    if hasattr(reader, "update"):
+        x, h = reader.update(x, branches, mult, add_row)
+        return x, Prepared(None, reader, h)
+    return ops.residual_norm(x, branches, mult, add_row=add_row)[0], None
+
+
+@BLOCKS.register("stream_pre_norm")
+class StreamPreNormBlock(Block):
+    """A norm in front of each sublayer, one after the other, on a 32-bit residual stream:
+        x <- x + mixer(norm1(x));  x <- x + ff(norm2(x))
+    ``feed_forward`` (with its norm) may be absent.  The branches hand over their last products' 32-bit sums; one
+    kernel adds a branch and writes the rows of the norm that reads the new stream (this block's second, the next
+    block's first, or the head's).  The norms are any that have ``update`` (``stream_rmsnorm``, ``stream_layernorm``);
+    the mixer must have ``mix`` and the feed-forward ``transform``."""
+
+    fuses_norm = True
+    can_defer_sum = True
+
+    def __init__(self, mixer_norm: PartSpec, mixer: PartSpec, ff_norm: PartSpec | None = None, feed_forward: PartSpec | None = None,
+                 shared: dict | None = None):
+        shared = shared if shared is not None else {}
+        if (ff_norm is None) != (feed_forward is None):
+            raise ValueError("a feed-forward and its norm come together")
+        self.mixer_norm = build_with_shared(NORMS, mixer_norm, shared)
+        self.mixer = build_with_shared(MIXERS, mixer, shared)
+        self.ff_norm = build_with_shared(NORMS, ff_norm, shared) if ff_norm is not None else None
+        self.feed_forward = build_with_shared(FEED_FORWARDS, feed_forward, shared) if feed_forward is not None else None
+        for n in (self.mixer_norm, self.ff_norm):
+            if n is not None and not hasattr(n, "update"):
+                raise ValueError("a stream_pre_norm block takes norms of a 32-bit stream")
+
+    def children(self) -> list[Part]:
+        return [c for c in (self.mixer_norm, self.mixer, self.ff_norm, self.feed_forward) if c is not None]
+
+    def tensor_specs(self) -> list[TensorSpec]:
+        return [s for c in self.children() for s in c.tensor_specs()]
+
+    def load(self, tensors: dict[str, torch.Tensor], placer: Placer) -> None:
+        for c in self.children():
+            c.load(tensors, placer)
+
+    def entry_norm(self):
+        return self.mixer_norm
+
+    def forward(self, x, ctx: StepContext, cache, state, rows, prepared: Prepared | None = None, next_norm=None,
+                defer_sum: bool = False):
+        """``defer_sum``: the last branch is not added; returns ``PendingSum`` for whoever runs next on the stream."""
+        if x.dtype != torch.float32:
+            raise TypeError("a stream_pre_norm block runs on a 32-bit stream (an embedding with stream_f32)")
+        if prepared is not None and prepared.norm is self.mixer_norm and prepared.normed is not None:
+            h = prepared.normed
+        else:
+            h = self.mixer_norm.forward(x)
+        branch = self.mixer.mix(h, ctx, cache, state, rows, out_f32=True)
+        if rows is not None:
+            x = ops.gather_rows(x, rows)
+        if self.feed_forward is not None:
+            x, made = _update_stream(x, (branch, None), self.ff_norm)
+            branch = self.feed_forward.transform(made.normed, out_f32=True)
+        if defer_sum:
+            return PendingSum(x, (branch, None), 1.0)
+        return _update_stream(x, (branch, None), next_norm)
+
+
+@CONNECTORS.register("add_row")
+class AddRow(Connector):
+    """x <- x + v on every row of a 32-bit stream, v one row of a learned matrix [rows, width] (what a run of layers that
+    is passed several times tells its passes apart by).  The row is kept in 32-bit.  It is added in the pass that adds
+    the branch of the block in front, where that was handed over unsummed, and writes the rows of the norm that reads
+    the new stream."""
+
+    updates_stream = True
+
+    def __init__(self, hidden_size: int, name: str, rows: int, row: int):
+        self.hidden_size, self.name, self.rows, self.row = int(hidden_size), name, int(rows), int(row)
+        if not 0 <= self.row < self.rows:
+            raise ValueError(f"row {row} of a matrix of {rows}")
+        self.vector: torch.Tensor | None = None
+
+    def tensor_specs(self) -> list[TensorSpec]:
+        return [TensorSpec(self.name, (self.rows, self.hidden_size), MATRIX)]
+
+    def load(self, tensors: dict[str, torch.Tensor], placer: Placer) -> None:
+        # (a place of its own for every row: the kernel that adds it reads 16 bytes at a time)
+        self.vector = placer.place(("row_f32", self.name, self.row), lambda: tensors[self.name][self.row].to(
+            torch.float32).clone().contiguous().to(placer.device))
+
+    def update(self, x: torch.Tensor, pending: "PendingSum | None", next_norm=None):
+        branches, mult = (pending.branches, pending.mult) if pending is not None else ((None, None), 1.0)
+        return _update_stream(x, branches, next_norm, mult, self.vector)
 
 
 @CONNECTORS.register("embedding_mix")

@@ -32,7 +32,9 @@ when they are placed, so that a query head is ``[rot_dim | key_dim]`` and a cach
 the value being the key's ``kv_rank`` elements behind the rotated part.  In the latent's space a head's
 query is ``[q_rot | W_uk,h^T q]`` (the matrix a head has an identity block), and the expansion of a cached
 key is ``[k_rot | W_uk,h c]`` (an identity block again, exact in either storage type).  With ``q_rank`` 0
-there is no query latent: ``q = W_q h``.  ``window``: a query sees itself and the window - 1 positions
+there is no query latent: ``q = W_q h``; with one, the heads' rotated parts come from ``W_uq`` and are turned behind it
+(``ops.rotate_heads_``).  A sink a head (``names["sink"]``) joins the softmax's denominator, and a gate per element
+(``names["g"]``, one more part of the product that reads h) multiplies the heads' results by its sigmoid.  ``window``: a query sees itself and the window - 1 positions
 before it; a portion then reads back and expands only the keys its queries see.
 
 Scores, softmax weights and norms are 32-bit arithmetic in either storage type; the kernels are
@@ -47,7 +49,7 @@ import torch
 
 from tokasaurus_amd.kernels import ops
 from tokasaurus_amd.kernels.upload import upload
-from tokasaurus_amd.parts.base import MATRIX, MIXERS, NORM_WEIGHT, POSITION_ENCODINGS, CacheNeed, CacheView, Mixer, PartSpec, StepContext, TensorSpec
+from tokasaurus_amd.parts.base import MIXERS, NORM_WEIGHT, POSITION_ENCODINGS, VECTOR, CacheNeed, CacheView, Mixer, PartSpec, StepContext, TensorSpec
 from tokasaurus_amd.parts.grouped_attention import tile_plan
 from tokasaurus_amd.parts.linear import Linear, Placer
 from tokasaurus_amd.parts.position import InterleavedRotary
@@ -63,21 +65,23 @@ class LatentAttention(Mixer):
         ([heads * value_dim, kv_rank]), o ([hidden, heads * value_dim]).  ``key_chunk``: in steps of
         few tokens a request's keys are cut at multiples of this many among workgroups (0: never).
         ``q_rank`` 0: no query latent; ``names`` has q ([heads * (key_dim + rot_dim), hidden]) instead of
-        dq, dq_norm, uq.  ``rot_dim`` (with ``q_rank`` 0): the rotated part of a head and of dkv's rows
-        (``kv_rank + rot_dim`` of them), turned by ``position`` (a rotation of pairs over at most rot_dim
-        elements).  ``window``: 0 for every earlier key."""
+        dq, dq_norm, uq.  ``rot_dim``: the rotated part of a head (behind its key_dim rows of q or uq) and of dkv's rows
+        (``kv_rank + rot_dim`` of them), turned by ``position`` (a rotation of neighbouring pairs over at most rot_dim
+        elements, or of the halves of all rot_dim).  ``window``: 0 for every earlier key.  Optional names: sink
+        ([heads], a score in the softmax's denominator that has no value), g ([heads * value_dim, hidden]: the heads'
+        results times sigmoid(W_g h), element by element)."""
         self.key_chunk = int(key_chunk)
         self.rot_dim, self.window = int(rot_dim), int(window)
         if self.rot_dim % 2 or self.rot_dim < 0:
             raise ValueError("the rotated part of a head has an even size")
-        if q_rank and self.rot_dim:
-            raise ValueError("a rotated part comes with queries projected directly (q_rank 0)")
         self.position = None
         if position is not None:
             shared = shared if shared is not None else {}
             self.position = shared.setdefault(("position", position), POSITION_ENCODINGS.build(position))
             if not isinstance(self.position, InterleavedRotary) or self.position.dims > self.rot_dim:
                 raise ValueError("latent_attention turns pairs of its rotated part: a rotation of pairs over at most rot_dim elements")
+            if self.position.pair_halves and self.position.dims != self.rot_dim:
+                raise ValueError("a rotation of halves turns the whole rotated part")
         self.heads_a_call = num_heads  # query heads one call of the plain attention kernel takes (set when the cache is checked)
         self.hidden_size, self.num_heads = hidden_size, num_heads
         self.key_dim, self.value_dim, self.q_rank, self.kv_rank = int(key_dim), int(value_dim), int(q_rank), int(kv_rank)
@@ -85,12 +89,15 @@ class LatentAttention(Mixer):
         self.names = dict(names)
         dr = self.rot_dim
         self.query_dim, self.cached_dim = dr + self.key_dim, dr + self.kv_rank  # a head's query, a cached key
-        if self.q_rank:
-            self.down = Linear(hidden_size, [names["dq"], names["dkv"]], [self.q_rank, self.kv_rank])
-            self.up_q = Linear(self.q_rank, [names["uq"]], [num_heads * self.key_dim])
-        else:  # [q | k_rot | c] in one product, the rotated parts leading (rows permuted when placed)
-            self.down = Linear(hidden_size, [names["q"], names["dkv"]], [num_heads * self.query_dim, self.cached_dim])
-            self.up_q = None
+        # one product for everything that reads h: [cq or q | k_rot | c | gate], the rotated parts leading (rows permuted
+        # when placed)
+        first, first_size = ("dq", self.q_rank) if self.q_rank else ("q", num_heads * self.query_dim)
+        self.gate_col = first_size + self.cached_dim if names.get("g") else None
+        gate = [names["g"]] if names.get("g") else []
+        self.down = Linear(hidden_size, [names[first], names["dkv"], *gate],
+                           [first_size, self.cached_dim] + [num_heads * self.value_dim] * len(gate))
+        self.up_q = Linear(self.q_rank, [names["uq"]], [num_heads * self.query_dim]) if self.q_rank else None
+        self.sink: torch.Tensor | None = None
         self.out = Linear(num_heads * self.value_dim, [names["o"]], [hidden_size])
         # all heads' keys and values of a cached key in one product (prompt portions)
         self.expand = Linear(self.kv_rank, [names["uk"], names["uv"]], [num_heads * self.key_dim, num_heads * self.value_dim])
@@ -108,6 +115,8 @@ class LatentAttention(Mixer):
             TensorSpec(n["dkv_norm"], (self.kv_rank,), NORM_WEIGHT)]
         if self.q_rank:
             specs += self.up_q.tensor_specs() + [TensorSpec(n["dq_norm"], (self.q_rank,), NORM_WEIGHT)]
+        if n.get("sink"):
+            specs.append(TensorSpec(n["sink"], (H,), VECTOR))
         return specs
 
     def cache_need(self) -> CacheNeed:
@@ -140,31 +149,40 @@ class LatentAttention(Mixer):
         self.c_norm_weight = f32(n["dkv_norm"])
         if self.position is not None:
             self.position.prepare(placer.device)
+        if n.get("sink"):
+            self.sink = f32(n["sink"])
         if self.q_rank:
-            for lin in (self.down, self.up_q, self.expand):
-                lin.load(tensors, placer)
             self.q_norm_weight = f32(n["dq_norm"])
+        if not dr:
+            for lin in (self.down, self.up_q, self.expand):
+                if lin is not None:
+                    lin.load(tensors, placer)
         else:
-            def rotated_first() -> torch.Tensor:
-                wq = tensors[n["q"]].to(placer.dtype).view(H, d + dr, -1)
-                wq = torch.cat([wq[:, d:], wq[:, :d]], dim=1).reshape(H * (d + dr), -1)
+            def rotated_first(name: str) -> torch.Tensor:  # the rows of every head, its rotated part moved to the front
+                w = tensors[name].to(placer.dtype).view(H, d + dr, -1)
+                return torch.cat([w[:, d:], w[:, :d]], dim=1).reshape(H * (d + dr), -1)
+
+            def stacked() -> torch.Tensor:
                 wkv = tensors[n["dkv"]].to(placer.dtype)
-                return torch.cat([wq, wkv[r:], wkv[:r]], dim=0).contiguous().to(placer.device)
+                parts = [tensors[n["dq"]].to(placer.dtype) if self.q_rank else rotated_first(n["q"]), wkv[r:], wkv[:r]]
+                if n.get("g"):
+                    parts.append(tensors[n["g"]].to(placer.dtype))
+                return torch.cat(parts, dim=0).contiguous().to(placer.device)
 
-            self.down.weight = placer.place(("rotated_first", n["q"], n["dkv"]), rotated_first)
-            if not dr:
-                self.expand.load(tensors, placer)
-            else:
-                def expansion() -> torch.Tensor:
-                    where = tensors[n["uk"]].device
-                    w = torch.zeros((H * (dr + d) + H * dv, dr + r), dtype=placer.dtype, device=where)
-                    keys = w[: H * (dr + d)].view(H, dr + d, dr + r)
-                    keys[:, :dr, :dr] = torch.eye(dr, dtype=placer.dtype, device=where)
-                    keys[:, dr:, dr:] = tensors[n["uk"]].to(placer.dtype).view(H, d, r)
-                    w[H * (dr + d) :, dr:] = tensors[n["uv"]].to(placer.dtype)
-                    return w.contiguous().to(placer.device)
+            self.down.weight = placer.place(("rotated_first", *self.down.names), stacked)
+            if self.q_rank:
+                self.up_q.weight = placer.place(("rotated_first", n["uq"]), lambda: rotated_first(n["uq"]).contiguous().to(placer.device))
 
-                self.expand_cached.weight = placer.place(("expansion_with_rotated_part", n["uk"], n["uv"]), expansion)
+            def expansion() -> torch.Tensor:
+                where = tensors[n["uk"]].device
+                w = torch.zeros((H * (dr + d) + H * dv, dr + r), dtype=placer.dtype, device=where)
+                keys = w[: H * (dr + d)].view(H, dr + d, dr + r)
+                keys[:, :dr, :dr] = torch.eye(dr, dtype=placer.dtype, device=where)
+                keys[:, dr:, dr:] = tensors[n["uk"]].to(placer.dtype).view(H, d, r)
+                w[H * (dr + d) :, dr:] = tensors[n["uv"]].to(placer.dtype)
+                return w.contiguous().to(placer.device)
+
+            self.expand_cached.weight = placer.place(("expansion_with_rotated_part", n["uk"], n["uv"]), expansion)
 
         def to_latent() -> torch.Tensor:
             where = tensors[n["uk"]].device
@@ -180,25 +198,28 @@ class LatentAttention(Mixer):
     def _attend(self, h: torch.Tensor, ctx: StepContext, cache: CacheView, rows: torch.Tensor | None) -> torch.Tensor:
         assert cache is not None and cache.writable, "latent attention keeps its latent in a cache of its own"
         H, r = self.num_heads, self.kv_rank
+        pos = self.position
+        rotation = dict(pair_halves=pos.pair_halves, rotation_scale=pos.magnitude) if pos is not None else {}
+        freq = pos.freq if pos is not None else None
+        down = self.down(h)
         if self.q_rank:
-            lat = self.down(h)  # [cq | c]
-            # both latents normed (each over its whole length), the key/value latent appended as key and as value
-            ops.qk_prepare(lat, ctx.positions, ctx.token_req, cache.block_table, self.q_norm_weight, self.c_norm_weight,
-                           self.norm_eps, None, cache.keys, cache.values, 1, 1, r, r, cache.page_size,
-                           query_dim=self.q_rank, values_are_keys=True)
-            cq = lat[:, : self.q_rank]
-            if lat.dtype != torch.float32 and (self.q_rank % 8 or lat.stride(0) % 8):
-                cq = torch.empty((lat.shape[0], self.q_rank), dtype=lat.dtype, device=lat.device).copy_(cq)
-            q = self.up_q(cq)  # [tokens, heads * key_dim]
-        else:
-            # [q | k_rot | c]: the latent normed, the rotated parts of every query head and of the key turned, the key
+            # [cq | k_rot | c]: both latents normed (each over its whole length), the key's rotated part turned, the key
             # [k_rot | c] appended and its latent part as the value
-            q = self.down(h)
-            pos = self.position
+            ops.qk_prepare(down, ctx.positions, ctx.token_req, cache.block_table, self.q_norm_weight, self.c_norm_weight,
+                           self.norm_eps, freq, cache.keys, cache.values, 1, 1, self.cached_dim, r, cache.page_size,
+                           query_dim=self.q_rank, values_are_keys=True, key_skip=self.rot_dim, rotate_queries=False, **rotation)
+            cq = down[:, : self.q_rank]
+            if down.dtype != torch.float32 and (self.q_rank % 8 or down.stride(0) % 8):
+                cq = torch.empty((down.shape[0], self.q_rank), dtype=down.dtype, device=down.device).copy_(cq)
+            q = self.up_q(cq)  # [tokens, heads * query_dim]
+            if freq is not None:
+                ops.rotate_heads_(q, ctx.positions, freq, H, self.query_dim, **rotation)
+        else:
+            # [q | k_rot | c]: the same with the rotated parts of every query head turned here
+            q = down
             ops.qk_prepare(q, ctx.positions, ctx.token_req, cache.block_table, None, self.c_norm_weight, self.norm_eps,
-                           pos.freq if pos is not None else None, cache.keys, cache.values, H, 1, self.cached_dim, r,
-                           cache.page_size, query_dim=self.query_dim, values_are_keys=True, key_skip=self.rot_dim,
-                           rotation_scale=pos.magnitude if pos is not None else 1.0)
+                           freq, cache.keys, cache.values, H, 1, self.cached_dim, r, cache.page_size, query_dim=self.query_dim,
+                           values_are_keys=True, key_skip=self.rot_dim, **rotation)
         # the requests that bring portions come first in a step; their tokens are the step's first rows
         portions = int(ctx.extras.get("num_portions", 0))
         first_single = ctx.host_q_start[portions] if portions else 0
@@ -208,6 +229,8 @@ class LatentAttention(Mixer):
                 o[first_single:] = self._over_latent(q[first_single:], ctx, cache, first_single, ctx.num_requests - portions)
         else:
             o = self._over_latent(q, ctx, cache, 0, None)
+        if self.gate_col is not None:
+            o = ops.sigmoid_gate(o, down[:, self.gate_col : self.gate_col + H * self.value_dim])
         return o if rows is None else ops.gather_rows(o, rows)
 
     def _over_latent(self, q: torch.Tensor, ctx: StepContext, cache: CacheView, first_row: int, last_requests: int | None) -> torch.Tensor:
@@ -222,7 +245,7 @@ class LatentAttention(Mixer):
             if last_requests is not None:  # a request of one token is one tile, whatever a tile holds
                 tile_req, tile_row0 = tile_req[tile_req.numel() - last_requests:], tile_row0[tile_row0.numel() - last_requests:]
             o = ops.attention_tile_f32(ql, cache.keys, cache.values, cache.block_table, ctx.q_start, ctx.kv_len,
-                                       tile_req, tile_row0, H, 1, dc, r, cache.page_size, gg, scale=self.scale, window=self.window,
+                                       tile_req, tile_row0, H, 1, dc, r, cache.page_size, gg, scale=self.scale, window=self.window, sink=self.sink,
                                        key_chunk=self.key_chunk, longest=ctx.extras.get("kv_bound", ctx.max_kv_len),
                                        first_row=first_row)
         else:
@@ -231,7 +254,8 @@ class LatentAttention(Mixer):
                 n = min(self.heads_a_call, H - h0)
                 part = ops.paged_attention_generic(ql[:, h0 * dc :], cache.keys, cache.values, cache.block_table,
                                                    ctx.token_req[first_row:], ctx.positions[first_row:], n, 1, dc, cache.page_size,
-                                                   window=self.window, scale=self.scale, value_dim=r)
+                                                   window=self.window, scale=self.scale, value_dim=r,
+                                                   sink=self.sink[h0 : h0 + n] if self.sink is not None else None)
                 if n == H:
                     o = part
                 else:
@@ -277,7 +301,7 @@ class LatentAttention(Mixer):
         ops.qk_prepare(kv, pos_d, req_d, table_d, None, None, 0.0, None, keys, values, 0, H, dk, dv, P)
         tile_req, tile_row0 = tile_plan(ctx, 16)
         return ops.attention_tile_f32(q, keys, values, table_d, ctx.q_start, ctx.kv_len, tile_req[:n_tiles], tile_row0[:n_tiles],
-                                      H, H, dk, dv, P, 1, scale=self.scale, window=self.window)
+                                      H, H, dk, dv, P, 1, scale=self.scale, window=self.window, sink=self.sink)
 
     def mix(self, h, ctx, cache, state, rows, out_f32: bool = False):
         return self.out(self._attend(h, ctx, cache, rows), out_f32=out_f32)

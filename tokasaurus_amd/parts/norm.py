@@ -66,8 +66,48 @@ class StreamRMSNorm(Norm):
         return isinstance(other, StreamRMSNorm) and (other.eps, other.unit_offset, other.size) == (self.eps, self.unit_offset, self.size)
 
     def forward(self, x: torch.Tensor) -> torch.Tensor:
-        return ops.residual_norm(x, weights=(self.weight, None), unit_offset=self.unit_offset, eps=self.eps,
-                                 out_dtype=self.out_dtype)[1]
+        return self.update(x)[1]
+
+    def update(self, x: torch.Tensor, branches: tuple = (None, None), mult: float = 1.0, add_row: torch.Tensor | None = None
+               ) -> tuple[torch.Tensor, torch.Tensor]:
+        """The stream with ``mult`` times the 32-bit ``branches`` and then one row for all (``add_row``) added, in place,
+        and this norm's rows of the result, in one pass."""
+        x, h, _ = ops.residual_norm(x, branches, mult, weights=(self.weight, None), unit_offset=self.unit_offset, eps=self.eps,
+                                    out_dtype=self.out_dtype, add_row=add_row)
+        return x, h
+
+
+@NORMS.register("stream_layernorm")
+class StreamLayerNorm(Norm):
+    """Layer norm with a weight and no bias on a residual stream that is kept in 32-bit whatever the storage type:
+    ``(x - m) / sqrt(mean((x - m)^2) + eps) * w`` with ``m = mean(x)``, computed in 32-bit and rounded once to the
+    storage type.  The weight is kept in 32-bit.  ``update`` as in ``StreamRMSNorm``."""
+
+    fusable_rms = False
+
+    def __init__(self, size: int, eps: float, name: str):
+        self.size = size
+        self.eps = float(eps)
+        self.name = name
+        self.weight: torch.Tensor | None = None
+        self.out_dtype: torch.dtype | None = None
+
+    def tensor_specs(self) -> list[TensorSpec]:
+        return [TensorSpec(self.name, (self.size,), NORM_WEIGHT)]
+
+    def load(self, tensors: dict[str, torch.Tensor], placer: Placer) -> None:
+        host = tensors[self.name]
+        self.weight = placer.place(("vector_f32", self.name), lambda: host.to(dtype=torch.float32).contiguous().to(placer.device))
+        self.out_dtype = placer.dtype
+
+    def forward(self, x: torch.Tensor) -> torch.Tensor:
+        return self.update(x)[1]
+
+    def update(self, x: torch.Tensor, branches: tuple = (None, None), mult: float = 1.0, add_row: torch.Tensor | None = None
+               ) -> tuple[torch.Tensor, torch.Tensor]:
+        x, h, _ = ops.residual_norm(x, branches, mult, weights=(self.weight, None), eps=self.eps, out_dtype=self.out_dtype,
+                                    add_row=add_row, center=True)
+        return x, h
 
 
 @NORMS.register("stream_cast")
