@@ -82,13 +82,13 @@ def parse() -> argparse.Namespace:
                    help="instead of the decode steps, a case that shapes of one length do not show (prints its own line): "
                         "chunked-prefill: one prompt of --context tokens in portions of --portion tokens; "
                         "mixed-decode: decode steps of --batch - 1 requests of --short tokens beside one of --context tokens")
-    p.add_argument("--design", default=None, choices=["kupuzen", "taborax", "sakevik", "sazilorn"],
+    p.add_argument("--design", default=None, choices=["kupuzen", "taborax", "sakevik", "sazilorn", "vekasun"],
                    help="instead of the decode steps: prefill and decode of this design at layer sizes of --design-sizes "
                         "beside the Llama shape of equal width, heads, feed-forward and layers (prints its own line)")
     p.add_argument("--design-sizes", default="1b,3b", help="which sizes of DESIGN_SIZES, comma separated")
-    p.add_argument("--design-beside", default=None, choices=["llama", "kupuzen", "taborax", "sakevik"],
+    p.add_argument("--design-beside", default=None, choices=["llama", "kupuzen", "taborax", "sakevik", "sazilorn"],
                    help="the model the --design comparison stands beside (by default the Llama shape; for sazilorn the Kupuzen "
-                        "of equal size, the closest existing design)")
+                        "of equal size and for vekasun the Taborax, the closest existing designs)")
     p.add_argument("--design-only", action="store_true", help="the --design comparison without its Llama half (for profiles)")
     p.add_argument("--design-layers", type=int, default=8, help="layers of both models in the --design comparison")
     p.add_argument("--design-context", type=int, default=4096, help="context at which the --design decode steps end")
@@ -433,7 +433,29 @@ def sazilorn_like(size: dict, layers: int) -> dict:
             "norm": {"eps": 1e-6}, "canon": {"taps": 4}, "layers": [kinds[i % 4] for i in range(layers)]}
 
 
-DESIGN_MODELS = {"kupuzen": kupuzen_like, "taborax": taborax_like, "sakevik": sakevik_like, "sazilorn": sazilorn_like}
+# A Vekasun of the same width, vocabulary and number of layer runs: latent attention (the Llama heads of the Llama size
+# beside a rotated part of 64, queries through a latent of 512, over a latent of 192: a cached key of 256) and two
+# state-space layers to every latent layer (twice the width in heads of 64, 128 rows of state, 8 groups, 4 taps); every
+# feed-forward a mixture whose eight chosen experts together have the Llama inner size (32 experts); two inner layers
+# are passed twice, so `layers` layer runs use `layers - 2` layers' weights.
+def vekasun_like(size: dict, layers: int) -> dict:
+    ll = size["llama"]
+    width = ll["hidden_size"]
+    d = width // ll["num_attention_heads"]
+    mixture = {"kind": "moe", "expert": {"ff": ll["intermediate_size"] // 8}, "router": {"experts": 32, "top": 8}}
+    latent = {"type": "latent_attention", "mlp": mixture, "mixer": {
+        "heads": ll["num_attention_heads"], "dim": d, "rot_dim": 64, "vdim": d, "q_rank": 512, "kv_rank": 192,
+        "scale": (d + 64) ** -0.5, "rot": {"base": ll["rope_theta"], "dims": 64}}}
+    mamba = {"type": "mamba2", "mlp": mixture, "mixer": {"heads": 2 * width // 64, "vdim": 64, "state": 128, "groups": 8, "conv": 4,
+                                                         "norm_groups": 8}}
+    distinct = max(layers - 2, 3)
+    return {"architecture": "Vekasun", "vocab": ll["vocab_size"], "width": width, "norm": {"eps": 1e-6}, "logit_scale": 0.5,
+            "loop": {"start": 1, "stop": 3, "times": 2}, "layers": [latent if i % 3 == 1 else mamba for i in range(distinct)]}
+
+
+DESIGN_MODELS = {"kupuzen": kupuzen_like, "taborax": taborax_like, "sakevik": sakevik_like, "sazilorn": sazilorn_like,
+                 "vekasun": vekasun_like}
+DESIGN_BESIDE = {"sazilorn": "kupuzen", "vekasun": "taborax"}  # the closest existing design where that is not the Llama shape
 
 
 def run_design(args) -> int:
@@ -441,7 +463,7 @@ def run_design(args) -> int:
     size, both with seeded random weights through the same runner and engine."""
     import torch
 
-    beside = args.design_beside or ("kupuzen" if args.design == "sazilorn" else "llama")
+    beside = args.design_beside or DESIGN_BESIDE.get(args.design, "llama")
     out = {"metric": f"prefill and decode of {args.design} beside the {beside} shape of equal size", "unit": "tokens/s",
            "dtype": "bf16" if args.dtype == "bfloat16" else "fp32", "layers": args.design_layers, "sizes": {}}
     batches = [int(b) for b in args.points.split(",") if b] or [1]

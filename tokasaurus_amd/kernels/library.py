@@ -47,8 +47,8 @@ _SIGNATURES: dict[str, dict[str, list]] = {
         "tk_short_conv": [c_int, _P, c_int, _P, c_int, _P, c_size_t, _P, _P, _P, _P] + [c_int] * 4 + [_P],
         "tk_gelu_glu": [c_int, _P, _P, c_int, c_int, _P],
         "tk_residual_norm": [c_int, _P, _P, _P, c_float, _P, _P, _P, _P, c_float, c_float, c_int, _P, _P, c_int, c_int, _P],
-        "tk_state_space": [_P, c_int, c_int, c_int, _P, _P, c_int, _P, _P, _P, _P, c_size_t, c_size_t, _P, _P, _P, _P, _P, _P] + [c_int] * 7 + [_P],
-        "tk_state_space_rec_width": [c_int] * 4,
+        "tk_state_space": [c_int, _P, c_int, c_int, c_int, _P, _P, c_int, _P, _P, _P, _P, c_size_t, c_size_t, _P, _P, _P, _P, _P, _P] + [c_int] * 7 + [_P],
+        "tk_state_space_token_bytes": [c_int] * 6,
         "tk_gate_group_norm": [c_int, _P, _P, c_int, _P, c_float, _P, c_int, c_int, c_int, _P],
         "tk_rotate_heads": [c_int, _P, c_int, _P, _P] + [c_int] * 5 + [c_float, _P],
         "tk_softcap": [_P, c_size_t, c_float, _P],

@@ -1354,14 +1354,16 @@ def state_space_sizes(heads: int, groups: int, state: int, value_dim: int, taps:
 def state_space(proj: torch.Tensor, x_off: int, dt_off: int, conv_w: torch.Tensor, conv_b: torch.Tensor, a_log: torch.Tensor,
                 dt_bias: torch.Tensor, d_skip: torch.Tensor, state: torch.Tensor, q_start: torch.Tensor, token_req: torch.Tensor,
                 slots: torch.Tensor, positions: torch.Tensor, heads: int, groups: int, state_dim: int, value_dim: int,
-                longest: int | None = None) -> torch.Tensor:
+                longest: int | None = None, storage: torch.dtype = torch.float32) -> torch.Tensor:
     """A selective state-space recurrence over every request's tokens of this step, from the 32-bit sums ``proj`` of one
     stacked product: columns x | B | C (heads * value_dim, groups * state_dim, groups * state_dim) from ``x_off`` on pass
     a causal convolution per channel (``conv_w`` [taps, channels] tap by tap, the last the current token's; ``conv_b``)
     and silu; dt = softplus(columns from ``dt_off`` on + ``dt_bias``), one a head; per head with the B and C of its group
     ``S <- exp(-exp(a_log) dt) S + dt B x^T``, ``y = S^T C + d_skip x``.  ``state`` [slots + 1, ``state_space_sizes``]
     (32-bit) is read and written in the requests' ``slots``.  ``longest``: the most tokens a request brings in this step
-    (the launch's form depends on it, the sums do not).  Returns y [tokens, heads * value_dim] in 32-bit."""
+    (the launch's form depends on it, and the order of the sums where portions go in chunks).  ``storage`` bfloat16: the
+    activated convolution is rounded to it, and long portions run as products on the matrix cores.  Returns
+    y [tokens, heads * value_dim] in 32-bit."""
     _gpu(proj, conv_w, conv_b, a_log, dt_bias, d_skip, state, q_start, token_req, slots, positions)
     H, G, N, dv = int(heads), int(groups), int(state_dim), int(value_dim)
     _need(proj.dim() == 2 and proj.dtype == torch.float32 and proj.stride(1) == 1, "state_space: 32-bit rows with unit inner stride")
@@ -1385,9 +1387,9 @@ def state_space(proj: torch.Tensor, x_off: int, dt_off: int, conv_w: torch.Tenso
     y = torch.empty((n, H * dv), dtype=torch.float32, device=proj.device)
     if n:
         longest = max(1, int(n if longest is None else longest))
-        rec = (torch.empty((n, load("core").tk_state_space_rec_width(H, G, N, dv)), dtype=torch.float32, device=proj.device)
-               if longest > 1 else None)
-        call("tk_state_space", proj.data_ptr(), proj.stride(0), int(x_off), int(dt_off), conv_w.data_ptr(), conv_b.data_ptr(), taps,
+        token_bytes = load("core").tk_state_space_token_bytes(dtype_code(storage), H, G, N, dv, longest)
+        rec = torch.empty((n * token_bytes,), dtype=torch.uint8, device=proj.device) if token_bytes else None
+        call("tk_state_space", dtype_code(storage), proj.data_ptr(), proj.stride(0), int(x_off), int(dt_off), conv_w.data_ptr(), conv_b.data_ptr(), taps,
              a_log.data_ptr(), dt_bias.data_ptr(), d_skip.data_ptr(), state.data_ptr(), state.stride(0), ring, q_start.data_ptr(),
              token_req.data_ptr(), slots.data_ptr(), positions.data_ptr(), rec.data_ptr() if rec is not None else None, y.data_ptr(), n,
              slots.numel(), H, G, N, dv, longest, _stream())

@@ -6,10 +6,12 @@ with a bias, and silu; ``dt <- softplus(dt + dt_bias)``, one number a head.  Per
 silu(z), every one of ``norm_groups`` equal parts is divided by its own root mean square, a weight multiplies the row,
 and the output projection follows.
 
-The products are in the storage type; their 32-bit sums go straight into the convolution, and everything from there to
-the norm's one rounding is 32-bit arithmetic in either storage type.  The state (the matrices and the convolution's last
+The products are in the storage type; their 32-bit sums go straight into the convolution, whose activated result is
+rounded once to the storage type; everything from there to the norm's one rounding is 32-bit arithmetic in either storage
+type.  The state (the matrices and the convolution's last
 inputs) is one row of 32-bit numbers in the request's slot, zero when a request takes the slot; a step of any cut
-continues from it with the sums of the token-by-token recurrence.
+continues from it.  Long portions in bfloat16 storage run as chunks of products on the matrix cores, with the same sums
+in another order.
 """
 
 from __future__ import annotations
@@ -70,7 +72,7 @@ class Mamba2(Mixer):
         proj = self.inp(h, out_f32=True)
         y = ops.state_space(proj, self.inner, self.inner + self.channels, self.conv_w, self.conv_b, self.a_log, self.dt_bias,
                             self.d_skip, state, ctx.q_start, ctx.token_req, ctx.slots, ctx.positions, self.num_heads, self.groups,
-                            self.state_dim, self.value_dim, longest=ctx.max_q_len)
+                            self.state_dim, self.value_dim, longest=ctx.max_q_len, storage=h.dtype)
         out = ops.gate_group_norm(y, proj[:, : self.inner], self.norm_w, self.norm_eps, self.norm_groups, h.dtype)
         return out if rows is None else ops.gather_rows(out, rows)
 
