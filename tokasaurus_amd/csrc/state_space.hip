@@ -20,10 +20,13 @@
 // In the first two the columns of S do not meet: a column is owned by SS_LANES neighbouring lanes that cut N between them and add up
 // through the wavefront's own data paths, always in the same order, so a token's result does not depend on how its
 // request's tokens were cut into steps or on what shares the batch.  The chunks' products add in another order.
+#include <math.h>
+
 #include "common.h"
 
 typedef float v4f __attribute__((ext_vector_type(4)));
 typedef __attribute__((ext_vector_type(8))) __bf16 bf16x8_t;
+typedef uint32_t u32x4 __attribute__((ext_vector_type(4)));
 
 #define SS_LANES 16
 #define SS_COLS 4    // value columns a wavefront owns
@@ -276,7 +279,7 @@ __global__ __launch_bounds__(4 * TK_WAVE) void ss_chunk_kernel(SsArgs a, const b
   if (first >= last) return;
   float* slot = a.state + (size_t)a.slots[r] * a.state_stride;
   ss_move_ring(a, slot, first, last, (blockIdx.z * gridDim.x + blockIdx.x) * blockDim.x + threadIdx.x, gridDim.x * gridDim.z * blockDim.x);
-  const int lane = threadIdx.x & (TK_WAVE - 1), wave = threadIdx.x / TK_WAVE;
+  const int lane = threadIdx.x & (TK_WAVE - 1), wave = __builtin_amdgcn_readfirstlane(threadIdx.x / TK_WAVE);
   const int col = lane & 15, c = lane >> 4;
   const int j0 = blockIdx.z * 16, j = j0 + col;
   const bool live = j < a.dv;
@@ -298,7 +301,7 @@ __global__ __launch_bounds__(4 * TK_WAVE) void ss_chunk_kernel(SsArgs a, const b
       }
   // what a thread brings of the next chunk: pieces of its rows of B and C, four numbers of x, and (first wavefront) a
   // token's step.  Tokens beyond the request's end repeat the last one's row and have no step and no decay.
-  uint4 pre[PER];
+  u32x4 pre[PER];
   bf16_t prex[4];
   float2 mine;
   auto ask = [&](int t0) {
@@ -306,7 +309,7 @@ __global__ __launch_bounds__(4 * TK_WAVE) void ss_chunk_kernel(SsArgs a, const b
     for (int k = 0; k < PER; ++k) {
       const int i = threadIdx.x + 256 * k, row = i / PIECES, piece = i % PIECES;
       const bf16_t* src = rec + (size_t)min(t0 + row, last - 1) * ld_rec + b_at;
-      pre[k] = *(const uint4*)(src + (piece < NROWS / 8 ? piece * 8 : a.G * NROWS + piece * 8 - NROWS));
+      pre[k] = *(const u32x4*)(src + (piece < NROWS / 8 ? piece * 8 : a.G * NROWS + piece * 8 - NROWS));
     }
 #pragma unroll
     for (int k = 0; k < 4; ++k) {
@@ -319,7 +322,7 @@ __global__ __launch_bounds__(4 * TK_WAVE) void ss_chunk_kernel(SsArgs a, const b
 #pragma unroll
     for (int k = 0; k < PER; ++k) {
       const int i = threadIdx.x + 256 * k, row = i / PIECES, piece = i % PIECES;
-      *(uint4*)(bc + row * LD + piece * 8) = pre[k];
+      *(u32x4*)(bc + row * LD + piece * 8) = pre[k];
     }
 #pragma unroll
     for (int k = 0; k < 4; ++k) {
@@ -373,7 +376,7 @@ __global__ __launch_bounds__(4 * TK_WAVE) void ss_chunk_kernel(SsArgs a, const b
     }
     {
       const float4 lt = *(const float4*)(l_lds + 16 * wave + 4 * c);
-      y[0] *= exp2f(lt.x); y[1] *= exp2f(lt.y); y[2] *= exp2f(lt.z); y[3] *= exp2f(lt.w);
+      y[0] *= __builtin_amdgcn_exp2f(lt.x); y[1] *= __builtin_amdgcn_exp2f(lt.y); y[2] *= __builtin_amdgcn_exp2f(lt.z); y[3] *= __builtin_amdgcn_exp2f(lt.w);
     }
     // y: what the chunk's own tokens give each other; the lane of token t holds tokens s = 16 T + 4 c + i
     const float l_t = l_lds[16 * wave + col], l_end = l_lds[SS_CHUNK - 1];
@@ -383,7 +386,7 @@ __global__ __launch_bounds__(4 * TK_WAVE) void ss_chunk_kernel(SsArgs a, const b
       const float4 ls = *(const float4*)(l_lds + 16 * T + 4 * c), ds = *(const float4*)(dt_lds + 16 * T + 4 * c);
       const float lv[4] = {ls.x, ls.y, ls.z, ls.w}, dv4[4] = {ds.x, ds.y, ds.z, ds.w};
 #pragma unroll
-      for (int i = 0; i < 4; ++i) ws[T][i] = exp2f(l_end - lv[i]) * dv4[i] * xv[T][i];
+      for (int i = 0; i < 4; ++i) ws[T][i] = __builtin_amdgcn_exp2f(l_end - lv[i]) * dv4[i] * xv[T][i];
       if (T > wave) continue;  // (the same for all lanes)
       v4f gm = (v4f){0.f, 0.f, 0.f, 0.f};
 #pragma unroll
@@ -392,7 +395,7 @@ __global__ __launch_bounds__(4 * TK_WAVE) void ss_chunk_kernel(SsArgs a, const b
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
         const bool seen = T < wave || 4 * c + i <= col;
-        const float w = seen ? gm[i] * (exp2f(l_t - lv[i]) * dv4[i]) : 0.f;
+        const float w = gm[i] * (__builtin_amdgcn_exp2f(seen ? l_t - lv[i] : -INFINITY) * dv4[i]);
         y = __builtin_amdgcn_mfma_f32_16x16x4f32(w, xv[T][i], y, 0, 0, 0);
       }
       if (T == wave) {
@@ -404,7 +407,7 @@ __global__ __launch_bounds__(4 * TK_WAVE) void ss_chunk_kernel(SsArgs a, const b
       }
     }
     // the state behind the chunk
-    const float keep = exp2f(l_end);
+    const float keep = __builtin_amdgcn_exp2f(l_end);
 #pragma unroll
     for (int p = 0; p < NP; ++p) {
       const int n = 32 * (wave + 4 * p) + 2 * col;
