@@ -9,7 +9,28 @@ head's state, dv the size of a head's value.
 
 from __future__ import annotations
 
+from contextlib import contextmanager
+
 import torch
+
+_round = False
+
+
+@contextmanager
+def rounding():
+    """Inside, what an engine with bfloat16 storage keeps in bfloat16 (rows behind norms, activations, queries, keys and
+    values) is rounded to it: a measure of what rounding alone does to a row, in the place of a tolerance."""
+    global _round
+    _round = True
+    try:
+        yield
+    finally:
+        _round = False
+
+
+def kept(x: torch.Tensor) -> torch.Tensor:
+    return x.float().bfloat16().to(x.dtype) if _round else x
+
 
 
 def rms(x: torch.Tensor, eps: float) -> torch.Tensor:
@@ -20,7 +41,7 @@ def rms(x: torch.Tensor, eps: float) -> torch.Tensor:
 def layer_norm(x: torch.Tensor, weight: torch.Tensor, eps: float) -> torch.Tensor:
     """(x - mean) / sqrt(mean((x - mean)^2) + eps) * weight over the last axis; no bias."""
     d = x - x.mean(-1, keepdim=True)
-    return d / torch.sqrt((d * d).mean(-1, keepdim=True) + eps) * weight
+    return kept(d / torch.sqrt((d * d).mean(-1, keepdim=True) + eps) * weight)
 
 
 def silu(z: torch.Tensor) -> torch.Tensor:
@@ -66,7 +87,7 @@ def state_space(x: torch.Tensor, B: torch.Tensor, C: torch.Tensor, dt: torch.Ten
 def gate_then_norm(y: torch.Tensor, z: torch.Tensor, weight: torch.Tensor, groups: int, eps: float) -> torch.Tensor:
     """y * silu(z), then every one of ``groups`` equal parts of a row over its own root mean square, times weight."""
     v = y * silu(z)
-    return rms(v.reshape(v.shape[0], groups, -1), eps).reshape(v.shape) * weight
+    return kept(rms(v.reshape(v.shape[0], groups, -1), eps).reshape(v.shape) * weight)
 
 
 def mamba2_mixer(h: torch.Tensor, w: dict, p: str, m: dict, eps: float) -> torch.Tensor:
@@ -74,7 +95,7 @@ def mamba2_mixer(h: torch.Tensor, w: dict, p: str, m: dict, eps: float) -> torch
     H, dv, N, G = int(m["heads"]), int(m["vdim"]), int(m["state"]), int(m["groups"])
     inner = H * dv
     z, u, dt = torch.split(h @ w[f"{p}.in"].T, [inner, inner + 2 * G * N, H], dim=-1)
-    u = silu(causal_convolution(u, w[f"{p}.conv"], w[f"{p}.conv.b"]))
+    u = kept(silu(causal_convolution(u, w[f"{p}.conv"], w[f"{p}.conv.b"])))
     x, B, C = torch.split(u, [inner, G * N, G * N], dim=-1)
     dt = softplus(dt + w[f"{p}.dt_bias"])
     y = state_space(x.reshape(T, H, dv), B.reshape(T, G, N), C.reshape(T, G, N), dt, w[f"{p}.A_log"], w[f"{p}.D"]).reshape(T, inner)
@@ -111,22 +132,22 @@ def latent_attention_mixer(h: torch.Tensor, w: dict, p: str, m: dict, eps: float
     T = h.shape[0]
     H, d, r, dv, rank = int(m["heads"]), int(m["dim"]), int(m["rot_dim"]), int(m["vdim"]), int(m["kv_rank"])
     base = float(m["rot"]["base"])
-    cq = rms(h @ w[f"{p}.dq"].T, eps) * w[f"{p}.dq.norm"]
+    cq = kept(rms(h @ w[f"{p}.dq"].T, eps) * w[f"{p}.dq.norm"])
     q = (cq @ w[f"{p}.uq"].T).view(T, H, d + r)
     down = h @ w[f"{p}.dkv"].T
-    c = rms(down[:, :rank], eps) * w[f"{p}.dkv.norm"]
+    c = kept(rms(down[:, :rank], eps) * w[f"{p}.dkv.norm"])
     k_rot = rotate_halves(down[:, rank:], base)
     k = torch.cat([(c @ w[f"{p}.uk"].T).view(T, H, d), k_rot[:, None, :].expand(T, H, r)], dim=-1)
     q = torch.cat([q[..., :d], rotate_halves(q[..., d:], base)], dim=-1)
-    o = sink_attention(q, k, (c @ w[f"{p}.uv"].T).view(T, H, dv), float(m["scale"]), w[f"{p}.sink"]).reshape(T, H * dv)
-    return (o * torch.sigmoid(h @ w[f"{p}.g"].T)) @ w[f"{p}.o"].T
+    o = sink_attention(kept(q), kept(k), (c @ w[f"{p}.uv"].T).view(T, H, dv), float(m["scale"]), w[f"{p}.sink"]).reshape(T, H * dv)
+    return kept(kept(o) * torch.sigmoid(h @ w[f"{p}.g"].T)) @ w[f"{p}.o"].T
 
 
 # --------------------------------------------------------------------------- feed-forward
 
 
 def expert(h: torch.Tensor, w: dict, p: str) -> torch.Tensor:
-    return (silu(h @ w[f"{p}.gate"].T) * (h @ w[f"{p}.up"].T)) @ w[f"{p}.down"].T
+    return kept(silu(h @ w[f"{p}.gate"].T) * (h @ w[f"{p}.up"].T)) @ w[f"{p}.down"].T
 
 
 def route(h: torch.Tensor, w: dict, p: str, r: dict) -> tuple[torch.Tensor, torch.Tensor]:

@@ -131,13 +131,29 @@ def row_error(row: torch.Tensor, ref: torch.Tensor) -> float:
     return float((row - ref).pow(2).mean().sqrt() / ref.pow(2).mean().sqrt().clamp_min(1e-9))
 
 
-def compare_rows(got: dict, plain: dict[str, torch.Tensor], tol: float) -> float:
+def rounding_limits(folder: Path, requests: dict[str, list[int]]) -> dict[tuple[str, int], float]:
+    """Three times what rounding alone does to every row.  A part of few numbers that nearly cancel in front of its norm
+    makes some rows of a small model move many times further than others."""
+    config, w = load_plain(folder)
+    out = {}
+    for rid, toks in requests.items():
+        exact = plain_vekasun.forward(toks, w, config)
+        with plain_vekasun.rounding():
+            rounded = plain_vekasun.forward(toks, w, config)
+        for pos in range(len(toks)):
+            out[rid, pos] = 3.0 * row_error(rounded[pos], exact[pos])
+    return out
+
+
+def compare_rows(got: dict, plain: dict[str, torch.Tensor], tol: float, limits: dict | None = None) -> float:
     """Every collected row against the plain row: the root mean square of the difference over the
-    vocabulary, relative to that of the plain row.  Names the first wrong (request, position)."""
+    vocabulary, relative to that of the plain row (a row may have a wider limit of its own).  Names the first wrong
+    (request, position)."""
     worst = 0.0
     for (rid, pos), row in sorted(got.items()):
         err = row_error(row, plain[rid][pos])
-        assert err <= tol, f"request {rid} position {pos}: relative error {err:.3e} (allowed {tol:.1e})"
+        allowed = max(tol, (limits or {}).get((rid, pos), 0.0))
+        assert err <= allowed, f"request {rid} position {pos}: relative error {err:.3e} (allowed {allowed:.1e})"
         worst = max(worst, err)
     return worst
 
