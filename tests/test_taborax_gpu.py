@@ -75,7 +75,7 @@ def test_router_kernel_against_the_plain_router():
             assert torch.allclose(gate.cpu().double(), torch.sigmoid(h @ gate_w.double()), atol=1e-5)
 
 
-@pytest.mark.parametrize("T, E, W, F, top", [(9, 5, 24, 12, 3), (70, 5, 24, 16, 3), (150, 7, 40, 72, 2), (33, 40, 64, 8, 4)])
+@pytest.mark.parametrize("T, E, W, F, top", [(9, 5, 24, 12, 3), (70, 5, 24, 16, 3), (150, 7, 40, 72, 2), (33, 40, 64, 8, 4), (500, 4, 200, 88, 3)])
 def test_expert_kernels_against_plain_experts(T, E, W, F, top):
     """The chosen experts' weighted sum with identity experts, an empty place and a shared expert: pair by pair
     for few tokens, sorted by expert into tiles on the matrix cores for many (bfloat16); experts that no token

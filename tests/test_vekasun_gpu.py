@@ -244,7 +244,7 @@ def test_router_with_sigmoid_scores():
     assert ids.cpu().tolist() == [[1, 2]] * 3 and torch.equal(wts.cpu(), torch.ones(3, 2))
 
 
-@pytest.mark.parametrize("T, E, W, F, top", [(9, 5, 24, 12, 3), (70, 5, 24, 16, 3), (150, 7, 40, 72, 2), (33, 40, 64, 8, 1), (260, 4, 128, 136, 4)])
+@pytest.mark.parametrize("T, E, W, F, top", [(9, 5, 24, 12, 3), (70, 5, 24, 16, 3), (150, 7, 40, 72, 2), (33, 40, 64, 8, 1), (260, 4, 128, 136, 4), (300, 3, 72, 200, 2)])
 def test_experts_that_read_weighted_rows(T, E, W, F, top):
     """sum of expert(weight * h): pair by pair for few tokens, sorted by expert into tiles for many (bfloat16); an
     identity expert, an empty place, an expert that nobody chose."""

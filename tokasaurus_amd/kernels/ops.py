@@ -1955,6 +1955,8 @@ def squared_relu_(x: torch.Tensor) -> torch.Tensor:
 # --------------------------------------------------------------------------
 
 GROUPED_TILE = 64  # slots a tile of the grouped matrix-core product (GG_TM of grouped_gemm.hip)
+GROUPED_LARGE_TILE = 128  # of the one that goes through local memory (GS_M)
+GROUPED_LARGE_FROM = 96  # pairs an expert has on average from which on the experts' products take the large tiles
 GROUPED_FROM_ROWS = 16  # rows above which the products of experts and of heads run in tiles on the matrix cores
 
 
@@ -1977,7 +1979,7 @@ def head_linear(x: torch.Tensor, w: torch.Tensor, out_f32: bool = False) -> torc
         # many rows: tiles of 32 rows on the matrix cores, the head as the tile's group
         tiles = -(-x.shape[0] // GROUPED_TILE)
         call("tk_grouped_gemm_bf16", x.data_ptr(), x.stride(0), None, None, None, tiles, heads, n_in, n_out, w.data_ptr(),
-             n_out * n_in, y.data_ptr(), y.stride(0), n_out, n_in, x.shape[0], 0, 1 if out_f32 else 0, None, None, _stream())
+             n_out * n_in, y.data_ptr(), y.stride(0), n_out, n_in, x.shape[0], 0, 1 if out_f32 else 0, None, None, GROUPED_TILE, _stream())
         return y
     if x.shape[0]:
         call("tk_head_linear", dtype_code(x.dtype), x.data_ptr(), x.stride(0), w.data_ptr(), y.data_ptr(), y.stride(0),
@@ -2044,19 +2046,20 @@ def expert_mix(h: torch.Tensor, w_gate_up: torch.Tensor, w_down: torch.Tensor, i
         return out
     if n > GROUPED_FROM_ROWS and _grouped_takes(h, w_gate_up, width) and ff % 8 == 0 and w_down.data_ptr() % 16 == 0:
         # many tokens: the pairs sorted by expert, every expert's rows in tiles on the matrix cores
-        max_tiles = -(-(n * top) // GROUPED_TILE) + experts
-        slots = max_tiles * GROUPED_TILE
-        book = torch.empty((2 * slots + max_tiles,), dtype=torch.int32, device=h.device)
+        tile = GROUPED_LARGE_TILE if n * top >= GROUPED_LARGE_FROM * experts else GROUPED_TILE
+        max_tiles = -(-(n * top) // tile) + experts
+        slots = max_tiles * tile
+        book = torch.empty((2 * slots + max_tiles + 1,), dtype=torch.int32, device=h.device)
         slot_pair, slot_token, tile_group = book[:slots], book[slots : 2 * slots], book[2 * slots :]
-        call("tk_expert_sort", ids.data_ptr(), n * top, top, experts, max_tiles, slot_pair.data_ptr(), slot_token.data_ptr(),
+        call("tk_expert_sort", ids.data_ptr(), n * top, top, experts, max_tiles, tile, slot_pair.data_ptr(), slot_token.data_ptr(),
              tile_group.data_ptr(), _stream())
         inter = torch.empty((slots, ff), dtype=h.dtype, device=h.device)
         call("tk_grouped_gemm_bf16", h.data_ptr(), h.stride(0), slot_token.data_ptr(), None, tile_group.data_ptr(), max_tiles, 0,
              0, 0, w_gate_up.data_ptr(), 2 * ff * width, inter.data_ptr(), ff, ff, width, slots, 1, 0, on_input,
-             slot_pair.data_ptr() if weights_on_input else None, _stream())
+             slot_pair.data_ptr() if weights_on_input else None, tile, _stream())
         y = torch.empty((n * top, width), dtype=h.dtype, device=h.device)
         call("tk_grouped_gemm_bf16", inter.data_ptr(), ff, None, slot_pair.data_ptr(), tile_group.data_ptr(), max_tiles, 0,
-             0, 0, w_down.data_ptr(), width * ff, y.data_ptr(), width, width, ff, slots, 0, 0, None, None, _stream())
+             0, 0, w_down.data_ptr(), width * ff, y.data_ptr(), width, width, ff, slots, 0, 0, None, None, tile, _stream())
         call("tk_expert_sum", h.data_ptr(), h.stride(0), y.data_ptr(), ids.data_ptr(), weights.data_ptr(),
              shared.data_ptr() if shared is not None else None, shared_gate.data_ptr() if shared is not None else None,
              out.data_ptr(), n, width, experts, top, unit, _stream())
