@@ -225,6 +225,28 @@ def test_rotation_of_a_head_s_leading_part(dtype):
     assert torch.allclose(near[:, 0], x[:, 0].double() * c - x[:, 1].double() * s, atol=tol * 3)
 
 
+@pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
+def test_a_matrix_a_head_with_a_rotation_and_a_gate(dtype):
+    """The leading part turned instead of multiplied by its identity block: the bits of turning first and multiplying
+    then; the result times a gate's sigmoid.  Neighbouring pairs and halves, a rotated part longer than a block of rows."""
+    torch.manual_seed(8)
+    for heads, dr, d, r, halves in ((3, 6, 10, 20, True), (2, 40, 8, 32, True), (2, 48, 8, 30, False), (1, 2, 3, 5, False)):
+        n = 7
+        w = torch.zeros(heads, dr + r, dr + d)
+        w[:, :dr, :dr] = torch.eye(dr)
+        w[:, dr:, dr:] = torch.randn(heads, r, d)
+        w, x, pos = w.to(dtype).cuda(), torch.randn(n, heads * (dr + d) + 3).to(dtype).cuda(), i32([0, 5, 9, 100, 3, 2, 1])
+        freq = torch.tensor([50.0 ** (-2.0 * i / dr) for i in range(dr // 2)], dtype=torch.float32).cuda()
+        want = ops.head_linear(ops.rotate_heads_(x.clone(), pos, freq, heads, dr + d, halves, 1.25), w)
+        got = ops.head_linear(x, w, positions=pos, freq=freq, pair_halves=halves, rotation_scale=1.25)
+        assert torch.equal(got, want)
+        gate = torch.randn(n, heads * (dr + r) + 5).to(dtype).cuda()[:, 5:]
+        gated = ops.head_linear(x, w, gate=gate).double().cpu()
+        ref = torch.einsum("thi,hoi->tho", x[:, : heads * (dr + d)].double().cpu().view(n, heads, dr + d), w.double().cpu()).reshape(n, -1)
+        tol = 1e-5 if dtype == torch.float32 else 2e-2
+        assert torch.allclose(gated, ref * torch.sigmoid(gate.double().cpu()), atol=tol, rtol=tol)
+
+
 def test_router_with_sigmoid_scores():
     torch.manual_seed(4)
     for experts, top, width in ((6, 3, 40), (1, 1, 16), (130, 8, 64), (5, 5, 24)):

@@ -102,6 +102,13 @@ __device__ __forceinline__ void shared_store16(void* p, uint16_t v) {
   __hip_atomic_store((uint16_t*)p, v, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
 }
 
+// What the lanes of one wavefront have written to local memory is there for its other lanes (a wavefront's accesses to
+// local memory are in order; the compiler must keep them so).
+__device__ __forceinline__ void wave_sync() {
+  __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+  __builtin_amdgcn_wave_barrier();
+}
+
 __device__ __forceinline__ float wave_sum(float v) {
 #pragma unroll
   for (int o = TK_WAVE / 2; o > 0; o >>= 1) v += __shfl_xor(v, o, TK_WAVE);

@@ -8,7 +8,8 @@
 //   tk_expert_gate_up    per (token, chosen expert): act(W_gate h) * (W_up h), of h or of weight * h
 //   tk_expert_combine    per token: sum of weight * W_down(...) over its experts, weight * h for an
 //                        identity expert, plus gate * (a shared expert's output)
-//   tk_head_linear       y[t, h, :] = W[h] x[t, h, :]: one matrix a head
+//   tk_head_linear       y[t, h, :] = W[h] x[t, h, :]: one matrix a head; optionally the leading part of a
+//                        head turned instead of multiplied, or the result times a sigmoid gate per element
 //   tk_squared_relu      x <- max(x, 0)^2, in place
 //
 // These kernels compute a row (a token, a pair) independently of every other row, with sums
@@ -95,15 +96,14 @@ __global__ __launch_bounds__(1024) void expert_route_kernel(
     }
   }
   __syncthreads();
-  // the rest is the work of one wavefront; the others only keep the barriers
-  const bool on = wave == 0;
-  if (on && SIGMOID) {
+  if (wave != 0) return;  // the rest is the work of one wavefront, whose lanes hand over through LDS in its own order
+  if (SIGMOID) {
     for (int e = lane; e < n_all; e += TK_WAVE) {
       const float z = score[e], s = 1.0f / (1.0f + expf(-z));
       score[e] = s;
       choice[e] = correction ? s + correction[e] : z;
     }
-  } else if (on) {
+  } else {
     float m = -INFINITY;
     for (int e = lane; e < n_all; e += TK_WAVE) m = fmaxf(m, score[e]);
     m = wave_max(m);
@@ -120,16 +120,15 @@ __global__ __launch_bounds__(1024) void expert_route_kernel(
       choice[e] = correction ? s + correction[e] : s;
     }
   }
-  __syncthreads();
-  const int per = n_all / groups;
-  if (on)
+  wave_sync();
+  if (keep < groups) {
+    const int per = n_all / groups;
     for (int g = lane; g < groups; g += TK_WAVE) {
       float best = -INFINITY;
       for (int e = g * per; e < (g + 1) * per; ++e) best = fmaxf(best, choice[e]);
       mark[g] = best;
     }
-  __syncthreads();
-  if (on && keep < groups)
+    wave_sync();
     for (int g = lane; g < groups; g += TK_WAVE) {
       int ahead = 0;  // groups that come before this one: a larger mark, or an equal one further left
       const float mine = mark[g];
@@ -137,35 +136,46 @@ __global__ __launch_bounds__(1024) void expert_route_kernel(
       if (ahead >= keep)
         for (int e = g * per; e < (g + 1) * per; ++e) choice[e] = -INFINITY;
     }
-  __syncthreads();
+    wave_sync();
+  }
+  // the `top` largest choices, ties to the left; with up to 64 experts a lane's choice stays in a register
+  const bool few = n_all <= TK_WAVE;
+  float mine = few && lane < n_all ? choice[lane] : -INFINITY;
+  float sum = 0.f;
   for (int r = 0; r < top; ++r) {
-    if (on) {
-      float best = -INFINITY;
-      int at = 0x7fffffff;
+    float best = -INFINITY;
+    int at = 0x7fffffff;
+    if (few) {
+      best = mine;
+      at = mine > -INFINITY ? lane : 0x7fffffff;
+    } else {
       for (int e = lane; e < n_all; e += TK_WAVE) {
         const float c = choice[e];
         if (c > best) { best = c; at = e; }
       }
-#pragma unroll
-      for (int o = TK_WAVE / 2; o > 0; o >>= 1) {
-        const float ob = __shfl_xor(best, o, TK_WAVE);
-        const int oa = __shfl_xor(at, o, TK_WAVE);
-        if (ob > best || (ob == best && oa < at)) { best = ob; at = oa; }
-      }
-      if (at == 0x7fffffff) at = -1;  // fewer open experts than places: the place stays empty
-      if (lane == 0) {
-        ids[(size_t)t * top + r] = at;
-        weights[(size_t)t * top + r] = at >= 0 ? score[at] : 0.f;
-        if (at >= 0) choice[at] = -INFINITY;
-      }
     }
-    __syncthreads();
+#pragma unroll
+    for (int o = TK_WAVE / 2; o > 0; o >>= 1) {
+      const float ob = __shfl_xor(best, o, TK_WAVE);
+      const int oa = __shfl_xor(at, o, TK_WAVE);
+      if (ob > best || (ob == best && oa < at)) { best = ob; at = oa; }
+    }
+    if (at == 0x7fffffff) at = -1;  // fewer open experts than places: the place stays empty
+    const float w = at >= 0 ? score[at] : 0.f;
+    sum += w;
+    if (lane == 0) {
+      ids[(size_t)t * top + r] = at;
+      weights[(size_t)t * top + r] = w;
+      if (at >= 0 && !few) choice[at] = -INFINITY;
+    }
+    if (few) {
+      if (lane == at) mine = -INFINITY;
+    } else {
+      wave_sync();
+    }
   }
-  if (norm_scale != 0.f && threadIdx.x == 0) {
-    float sum = 0.f;
-    for (int r = 0; r < top; ++r) sum += weights[(size_t)t * top + r];
+  if (norm_scale != 0.f && lane == 0)  // (the lane reads back what it wrote)
     for (int r = 0; r < top; ++r) weights[(size_t)t * top + r] = weights[(size_t)t * top + r] / (sum + 1e-20f) * norm_scale;
-  }
 }
 
 TK_API int tk_expert_route(int dt, const void* h, int h_stride, const void* w_router, const float* correction,
@@ -307,40 +317,75 @@ TK_API int tk_expert_combine(int dt, const void* h, int h_stride, const void* in
 // --------------------------------------------------------------------------
 // y[t, hd * n_out + o] = sum_i W[hd][o][i] * x[t, hd * n_in + i]: a matrix a head.  y is T or 32-bit.
 // Workgroup (token, head, block of HL_ROWS outputs).
+// `rot` > 0 (for a matrix whose leading rot x rot block is the identity, with zeros beside and below it): the leading
+// rot outputs of a head are its leading inputs turned by position * freq[i], pairs (i, i + rot/2) with `pair_half` and
+// (2i, 2i + 1) without, cosine and sine times rot_scale, rounded as the inputs are.
+// `gate` (or null): y[t, hd * n_out + o] is multiplied by sigmoid(gate[t, hd * n_out + o]) before its one rounding.
 // --------------------------------------------------------------------------
 #define HL_ROWS 32
+template <typename T>
+struct HeadExtra {
+  const int* positions;
+  const float* freq;
+  int rot, pair_half;
+  float rot_scale;
+  const T* gate;
+  int gate_stride;
+};
 template <typename T, typename O>
 __global__ __launch_bounds__(256) void head_linear_kernel(const T* __restrict__ x, int x_stride, const T* __restrict__ w,
-                                                          O* __restrict__ y, int y_stride, int n_in, int n_out) {
+                                                          O* __restrict__ y, int y_stride, int n_in, int n_out, HeadExtra<T> ex) {
   const int t = blockIdx.x, hd = blockIdx.y;
   const int lane = threadIdx.x & (TK_WAVE - 1), wave = threadIdx.x / TK_WAVE, nwaves = blockDim.x / TK_WAVE;
   const T* row = x + (size_t)t * x_stride + (size_t)hd * n_in;
   const T* wh = w + (size_t)hd * n_out * n_in;
+  O* dst = y + (size_t)t * y_stride + (size_t)hd * n_out;
   const int o0 = blockIdx.z * HL_ROWS;
-  for (int o = o0 + wave; o < min(o0 + HL_ROWS, n_out); o += nwaves) {
-    const float d = wave_dot<T>(wh + (size_t)o * n_in, row, n_in);
-    if (lane == 0) y[(size_t)t * y_stride + (size_t)hd * n_out + o] = from_f32<O>(d);
+  if (o0 < ex.rot) {  // this block's turned outputs, a thread a pair that begins here
+    const int half = ex.rot / 2;
+    for (int i = threadIdx.x; i < half; i += blockDim.x) {
+      const int e0 = ex.pair_half ? i : 2 * i, e1 = ex.pair_half ? i + half : 2 * i + 1;
+      if (e0 < o0 || e0 >= o0 + HL_ROWS) continue;
+      float sn, cs, u = to_f32<T>(row[e0]), v = to_f32<T>(row[e1]);
+      sincosf(__fmul_rn((float)ex.positions[t], ex.freq[i]), &sn, &cs);
+      rotate_pair(u, v, cs * ex.rot_scale, sn * ex.rot_scale, u, v);
+      dst[e0] = from_f32<O>(round_to<T>(u));
+      dst[e1] = from_f32<O>(round_to<T>(v));
+    }
+  }
+  for (int o = max(o0, ex.rot) + wave; o < min(o0 + HL_ROWS, n_out); o += nwaves) {
+    float d = wave_dot<T>(wh + (size_t)o * n_in, row, n_in);
+    if (lane == 0) {
+      if (ex.gate) d /= 1.0f + expf(-to_f32<T>(ex.gate[(size_t)t * ex.gate_stride + (size_t)hd * n_out + o]));
+      dst[o] = from_f32<O>(d);
+    }
   }
 }
 
 TK_API int tk_head_linear(int dt, const void* x, int x_stride, const void* w, void* y, int y_stride, int out_f32,
-                          int tokens, int heads, int n_in, int n_out, hipStream_t stream) {
+                          int tokens, int heads, int n_in, int n_out, const int* positions, const float* freq, int rot,
+                          int pair_half, float rot_scale, const void* gate, int gate_stride, hipStream_t stream) {
   TK_REQUIRE(tokens >= 0 && heads > 0 && n_in > 0 && n_out > 0 && x_stride >= heads * n_in && y_stride >= heads * n_out,
              "head_linear: bad sizes tokens=%d heads=%d in=%d out=%d strides %d %d", tokens, heads, n_in, n_out, x_stride,
              y_stride);
   TK_REQUIRE(x && w && y, "head_linear: a pointer is missing");
+  TK_REQUIRE(rot >= 0 && rot % 2 == 0 && rot <= n_in && rot <= n_out && (rot == 0 || (positions && freq)),
+             "head_linear: %d turned elements of heads of %d and %d", rot, n_in, n_out);
+  TK_REQUIRE(!gate || gate_stride >= heads * n_out, "head_linear: the gate's rows are too short");
   if (tokens == 0) return 0;
   const dim3 grid(tokens, heads, (n_out + HL_ROWS - 1) / HL_ROWS);
   TK_REQUIRE(grid.y < 65536 && grid.z < 65536, "head_linear: too many heads or outputs");
+  const HeadExtra<float> ef{positions, freq, rot, pair_half, rot_scale, (const float*)gate, gate_stride};
+  const HeadExtra<bf16_t> eb{positions, freq, rot, pair_half, rot_scale, (const bf16_t*)gate, gate_stride};
   if (dt == TK_F32)
     hipLaunchKernelGGL((head_linear_kernel<float, float>), grid, dim3(256), 0, stream, (const float*)x, x_stride,
-                       (const float*)w, (float*)y, y_stride, n_in, n_out);
+                       (const float*)w, (float*)y, y_stride, n_in, n_out, ef);
   else if (out_f32)
     hipLaunchKernelGGL((head_linear_kernel<bf16_t, float>), grid, dim3(256), 0, stream, (const bf16_t*)x, x_stride,
-                       (const bf16_t*)w, (float*)y, y_stride, n_in, n_out);
+                       (const bf16_t*)w, (float*)y, y_stride, n_in, n_out, eb);
   else
     hipLaunchKernelGGL((head_linear_kernel<bf16_t, bf16_t>), grid, dim3(256), 0, stream, (const bf16_t*)x, x_stride,
-                       (const bf16_t*)w, (bf16_t*)y, y_stride, n_in, n_out);
+                       (const bf16_t*)w, (bf16_t*)y, y_stride, n_in, n_out, eb);
   TK_CHECK_LAUNCH("head_linear");
   return 0;
 }

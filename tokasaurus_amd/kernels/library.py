@@ -65,7 +65,7 @@ _SIGNATURES: dict[str, dict[str, list]] = {
         "tk_expert_route": [c_int, _P, c_int, _P, _P, _P] + [c_int] * 6 + [_P, _P, _P, c_float, c_int, _P],
         "tk_expert_gate_up": [c_int, _P, c_int, _P, _P, _P, _P] + [c_int] * 5 + [_P],
         "tk_expert_combine": [c_int, _P, c_int, _P, _P, _P, _P, _P, _P, _P] + [c_int] * 6 + [_P],
-        "tk_head_linear": [c_int, _P, c_int, _P, _P, c_int, c_int] + [c_int] * 4 + [_P],
+        "tk_head_linear": [c_int, _P, c_int, _P, _P, c_int, c_int] + [c_int] * 4 + [_P, _P, c_int, c_int, c_float, _P, c_int, _P],
         "tk_squared_relu": [c_int, _P, c_size_t, _P],
         "tk_attention_tile_f32": [c_int, _P, c_int, _P, c_int, _P, _P, _P, c_int, _P, _P, _P, _P] + [c_int] * 7
         + [c_float, _P, _P, c_int, c_int, c_int, c_int, _P, _P, c_int, _P, c_int, c_float, _P, c_int, _P, _P],

@@ -1967,23 +1967,44 @@ def _grouped_takes(x: torch.Tensor, w: torch.Tensor, inner: int) -> bool:
             and w.data_ptr() % 16 == 0)
 
 
-def head_linear(x: torch.Tensor, w: torch.Tensor, out_f32: bool = False) -> torch.Tensor:
+def head_linear_is_fused(x: torch.Tensor, w: torch.Tensor) -> bool:
+    """Whether ``head_linear`` takes these rows in its own kernel, with a rotation or a gate in it (else in tiles on the
+    matrix cores, and the caller rotates and gates in passes of their own)."""
+    return not (x.shape[0] > GROUPED_FROM_ROWS and _grouped_takes(x, w, w.shape[2]))
+
+
+def head_linear(x: torch.Tensor, w: torch.Tensor, out_f32: bool = False, positions: torch.Tensor | None = None,
+                freq: torch.Tensor | None = None, pair_halves: bool = False, rotation_scale: float = 1.0,
+                gate: torch.Tensor | None = None) -> torch.Tensor:
     """y[t, h, :] = w[h] x[t, h, :] for w [heads, out, in] and the leading heads * in columns of
-    the rows of x; returns [tokens, heads * out] in x's type, or 32-bit sums with ``out_f32``."""
-    _gpu(x, w)
+    the rows of x; returns [tokens, heads * out] in x's type, or 32-bit sums with ``out_f32``.  Where
+    ``head_linear_is_fused``: with ``freq`` (and ``positions``) the leading 2 * len(freq) outputs of a head are its leading
+    inputs turned as ``rotate_heads_`` turns them (for a matrix with an identity block there); with ``gate``
+    [tokens, heads * out] (rows a stride apart) the result is multiplied by its sigmoid."""
+    _gpu(x, w, positions, freq, gate)
     _need(w.dim() == 3 and w.is_contiguous() and w.dtype == x.dtype, "head_linear: weights contiguous [heads, out, in] of the rows' type")
     heads, n_out, n_in = w.shape
     _need(x.dim() == 2 and x.stride(1) == 1 and x.shape[1] >= heads * n_in, "head_linear: rows of unit inner stride that hold heads * in columns")
     y = torch.empty((x.shape[0], heads * n_out), dtype=torch.float32 if out_f32 else x.dtype, device=x.device)
-    if x.shape[0] > GROUPED_FROM_ROWS and _grouped_takes(x, w, n_in):
+    if not head_linear_is_fused(x, w):
+        _need(freq is None and gate is None, "head_linear: so many rows are rotated and gated in passes of their own")
         # many rows: tiles of 32 rows on the matrix cores, the head as the tile's group
         tiles = -(-x.shape[0] // GROUPED_TILE)
         call("tk_grouped_gemm_bf16", x.data_ptr(), x.stride(0), None, None, None, tiles, heads, n_in, n_out, w.data_ptr(),
              n_out * n_in, y.data_ptr(), y.stride(0), n_out, n_in, x.shape[0], 0, 1 if out_f32 else 0, None, None, GROUPED_TILE, _stream())
         return y
+    if freq is not None:
+        _i32(positions, "positions")
+        _need(positions.numel() == x.shape[0] and freq.dim() == 1 and freq.dtype == torch.float32 and freq.is_contiguous(),
+              "head_linear: one position a row, frequencies contiguous float32")
+    _need(gate is None or (gate.shape == y.shape and gate.dtype == x.dtype and gate.stride(1) == 1),
+          "head_linear: a gate of the result's shape and the rows' type")
     if x.shape[0]:
         call("tk_head_linear", dtype_code(x.dtype), x.data_ptr(), x.stride(0), w.data_ptr(), y.data_ptr(), y.stride(0),
-             1 if (out_f32 and x.dtype != torch.float32) else 0, x.shape[0], heads, n_in, n_out, _stream())
+             1 if (out_f32 and x.dtype != torch.float32) else 0, x.shape[0], heads, n_in, n_out,
+             positions.data_ptr() if freq is not None else None, freq.data_ptr() if freq is not None else None,
+             2 * freq.numel() if freq is not None else 0, 1 if pair_halves else 0, float(rotation_scale),
+             gate.data_ptr() if gate is not None else None, gate.stride(0) if gate is not None else 0, _stream())
     return y
 
 

@@ -202,6 +202,8 @@ class LatentAttention(Mixer):
         rotation = dict(pair_halves=pos.pair_halves, rotation_scale=pos.magnitude) if pos is not None else {}
         freq = pos.freq if pos is not None else None
         down = self.down(h)
+        to_turn = False  # whether the queries' rotated parts are still to be turned
+        gate = down[:, self.gate_col : self.gate_col + H * self.value_dim] if self.gate_col is not None else None
         if self.q_rank:
             # [cq | k_rot | c]: both latents normed (each over its whole length), the key's rotated part turned, the key
             # [k_rot | c] appended and its latent part as the value
@@ -212,8 +214,7 @@ class LatentAttention(Mixer):
             if down.dtype != torch.float32 and (self.q_rank % 8 or down.stride(0) % 8):
                 cq = torch.empty((down.shape[0], self.q_rank), dtype=down.dtype, device=down.device).copy_(cq)
             q = self.up_q(cq)  # [tokens, heads * query_dim]
-            if freq is not None:
-                ops.rotate_heads_(q, ctx.positions, freq, H, self.query_dim, **rotation)
+            to_turn = freq is not None
         else:
             # [q | k_rot | c]: the same with the rotated parts of every query head turned here
             q = down
@@ -223,22 +224,32 @@ class LatentAttention(Mixer):
         # the requests that bring portions come first in a step; their tokens are the step's first rows
         portions = int(ctx.extras.get("num_portions", 0))
         first_single = ctx.host_q_start[portions] if portions else 0
-        if portions and ops.attention_tile_f32_fits(H, H, self.query_dim, self.value_dim, cache.page_size):
+        expanded = bool(portions) and ops.attention_tile_f32_fits(H, H, self.query_dim, self.value_dim, cache.page_size)
+        turn = dict(positions=ctx.positions, freq=freq, **rotation) if to_turn else {}
+        if expanded:
+            if to_turn:
+                ops.rotate_heads_(q, ctx.positions, freq, H, self.query_dim, **rotation)
             o = self._over_expanded(q, ctx, cache, portions)
             if first_single < ctx.num_tokens:
                 o[first_single:] = self._over_latent(q[first_single:], ctx, cache, first_single, ctx.num_requests - portions)
+            if gate is not None:
+                o = ops.sigmoid_gate(o, gate)
         else:
-            o = self._over_latent(q, ctx, cache, 0, None)
-        if self.gate_col is not None:
-            o = ops.sigmoid_gate(o, down[:, self.gate_col : self.gate_col + H * self.value_dim])
+            o = self._over_latent(q, ctx, cache, 0, None, turn, gate)
         return o if rows is None else ops.gather_rows(o, rows)
 
-    def _over_latent(self, q: torch.Tensor, ctx: StepContext, cache: CacheView, first_row: int, last_requests: int | None) -> torch.Tensor:
+    def _over_latent(self, q: torch.Tensor, ctx: StepContext, cache: CacheView, first_row: int, last_requests: int | None,
+                     turn: dict | None = None, gate: torch.Tensor | None = None) -> torch.Tensor:
         """Attention in the latent's space for the step's rows from ``first_row`` on (``q`` holds those
         rows), which belong to the step's last ``last_requests`` requests, one token each (None: all
-        rows of all requests)."""
+        rows of all requests).  ``turn`` (a rotation, for ``ops.head_linear``) and ``gate``: what is still to be done to
+        the queries and to the results: in the products with a matrix a head where they can (few rows), else in passes
+        of their own."""
         H, r, dc = self.num_heads, self.kv_rank, self.cached_dim
-        ql = ops.head_linear(q, self.to_latent)  # [rows, heads * cached_dim]
+        if turn and not ops.head_linear_is_fused(q, self.to_latent):
+            ops.rotate_heads_(q, turn["positions"], turn["freq"], H, self.query_dim, turn["pair_halves"], turn["rotation_scale"])
+            turn = None
+        ql = ops.head_linear(q, self.to_latent, **(turn or {}))  # [rows, heads * cached_dim]
         if ops.attention_tile_f32_fits(H, 1, dc, r, cache.page_size):
             gg = ops.attention_tile_heads(H, ctx.max_q_len if last_requests is None else 1)
             tile_req, tile_row0 = tile_plan(ctx, 16 // gg)
@@ -260,7 +271,9 @@ class LatentAttention(Mixer):
                     o = part
                 else:
                     o[:, h0 * r : (h0 + n) * r] = part
-        return ops.head_linear(o, self.from_latent)  # [rows, heads * value_dim]
+        if gate is None or ops.head_linear_is_fused(o, self.from_latent):
+            return ops.head_linear(o, self.from_latent, gate=gate)  # [rows, heads * value_dim]
+        return ops.sigmoid_gate(ops.head_linear(o, self.from_latent), gate)
 
     def _over_expanded(self, q: torch.Tensor, ctx: StepContext, cache: CacheView, portions: int) -> torch.Tensor:
         """Attention over expanded keys and values for the tokens of the step's first ``portions``
