@@ -4,8 +4,8 @@ Layers (run entries) whose caches have equal needs form a *group*: one pool of
 page ids and, per request, one block table that every layer of the group uses
 (the reference has a single such group: one table per sequence shared by all
 layers, tokasaurus/manager/types.py:46, tokasaurus/model/llama.py:675-691).
-A group whose layers read only a window of keys gives pages back as soon as the
-window has passed them; a full group gives pages back when the request ends.
+A group whose layers read only a window (or a section) of keys gives pages back as soon as
+that has passed them; a full group gives pages back when the request ends.
 Token ``pos`` of a request lives in page ``table[pos // P]`` at offset ``pos % P``
 (tokasaurus/manager/input_building.py:138-148).
 
@@ -62,6 +62,8 @@ def plan_groups(needs: list, cache_of: list[int | None]) -> tuple[list[CacheGrou
             owner_need = theirs[j]
             if (owner_need.num_kv_heads, owner_need.head_dim, owner_need.value_size) != (need.num_kv_heads, need.head_dim, need.value_size):
                 raise ValueError(f"run entry {i} cannot read the cache of entry {owner}: head layout differs")
+            if need.section != owner_need.section and not owner_need.keeps_all:
+                raise ValueError(f"run entry {i} reads other keys than entry {owner} keeps")
             if owner_need.window and (not need.window or need.window > owner_need.window):
                 raise ValueError(f"run entry {i} reads further back than entry {owner} keeps keys")
             places.append((group_of[owner_need], index[(owner, j)][1]))
@@ -179,11 +181,10 @@ class CacheManager:
         rc.num_tokens = new_len
         P = self.page_size
         for g, grp in enumerate(self.groups):
-            w = grp.need.window
-            if not w:
+            if grp.need.keeps_all:
                 continue
-            # the next query sits at position >= new_len and reads from new_len - w + 1 on
-            first_needed = max(0, new_len - w + 1) // P
+            # the next query sits at position >= new_len
+            first_needed = grp.need.first_read(new_len) // P
             table = rc.tables[g]
             gone = []
             for b in range(rc.first_held[g], min(first_needed, len(table))):

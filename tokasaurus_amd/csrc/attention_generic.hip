@@ -10,7 +10,8 @@
 //
 //   K pages: [page][kv head][d / 8][P][8]   V pages: [page][kv head][P / 4][d][4]
 //   (key_offset and value_offset of common.h); block_table[req][pos / P] is the page of a position.
-// A query at position p sees positions max(0, p - window + 1) .. p (window <= 0: all).
+// A query at position p sees positions max(0, p - window + 1) .. p (window <= 0: all), or with `section` > 0 those of its own
+// section, p / section * section .. p.
 // Keys have d elements a head and values dv (dv = d in most models).  `sink` (null, or one
 // 32-bit number a query head): exp(sink) is added once to the softmax's denominator; it has no
 // key and no value.  `score_bias` (null, or one 32-bit number a query head): the weights are no
@@ -27,7 +28,7 @@ __global__ __launch_bounds__(AG_THREADS) void paged_attention_generic_kernel(
     const T* __restrict__ q, int q_stride, T* __restrict__ out, int out_stride,
     const T* __restrict__ kcache, const T* __restrict__ vcache,
     const int* __restrict__ block_table, int table_stride, const int* __restrict__ token_req,
-    const int* __restrict__ positions, int nq, int nkv, int d, int dv, int P, int window, float scale,
+    const int* __restrict__ positions, int nq, int nkv, int d, int dv, int P, int window, int section, float scale,
     const float* __restrict__ sink, const float* __restrict__ score_bias, float softcap,
     const int* __restrict__ bucket_of, int far, const float* __restrict__ rel) {
   extern __shared__ float smem[];
@@ -36,7 +37,7 @@ __global__ __launch_bounds__(AG_THREADS) void paged_attention_generic_kernel(
   const int tid = threadIdx.x;
   const int lane = tid & (TK_WAVE - 1), wave = tid / TK_WAVE;
   const int pos = positions[t];
-  const int lo = window > 0 ? max(0, pos - window + 1) : 0;
+  const int lo = section > 0 ? pos / section * section : (window > 0 ? max(0, pos - window + 1) : 0);
   const int* table = block_table + (size_t)token_req[t] * table_stride;
 
   float* qs = smem;                    // [group][d]
@@ -158,12 +159,12 @@ template <typename T, int CH>
 static void ag_launch(const void* q, int q_stride, void* out, int out_stride, const void* kcache,
                       const void* vcache, const int* block_table, int table_stride,
                       const int* token_req, const int* positions, int n_tokens, int nq, int nkv,
-                      int d, int dv, int P, int window, float scale, const float* sink, const float* score_bias,
+                      int d, int dv, int P, int window, int section, float scale, const float* sink, const float* score_bias,
                       float softcap, const int* bucket_of, int far, const float* rel, hipStream_t stream) {
   hipLaunchKernelGGL((paged_attention_generic_kernel<T, CH>), dim3(n_tokens, nkv),
                      dim3(AG_THREADS), ag_smem_bytes(nq / nkv, d, dv, CH), stream, (const T*)q,
                      q_stride, (T*)out, out_stride, (const T*)kcache, (const T*)vcache,
-                     block_table, table_stride, token_req, positions, nq, nkv, d, dv, P, window, scale, sink, score_bias,
+                     block_table, table_stride, token_req, positions, nq, nkv, d, dv, P, window, section, scale, sink, score_bias,
                      softcap, bucket_of, far, rel);
 }
 
@@ -184,9 +185,10 @@ TK_API int tk_paged_attention_generic(int dt, const void* q, int q_stride, void*
                                           int out_stride, const void* kcache, const void* vcache,
                                           const int* block_table, int table_stride,
                                           const int* token_req, const int* positions, int n_tokens,
-                                          int nq, int nkv, int d, int dv, int P, int window, float scale,
+                                          int nq, int nkv, int d, int dv, int P, int window, int section, float scale,
                                           const float* sink, const float* score_bias, float softcap,
                                           const int* bucket_of, int far, const float* rel, hipStream_t stream) {
+  TK_REQUIRE(section <= 0 || window <= 0, "paged_attention: a window or sections, not both");
   TK_REQUIRE(!rel || (bucket_of && far >= 0), "paged_attention: a bias by distance needs its table of buckets");
   TK_REQUIRE(n_tokens >= 0 && nq > 0 && nkv > 0 && d > 0 && dv > 0 && P > 0 && nq % nkv == 0,
              "paged_attention: bad sizes tokens=%d nq=%d nkv=%d d=%d dv=%d P=%d", n_tokens, nq, nkv, d, dv,
@@ -205,7 +207,7 @@ TK_API int tk_paged_attention_generic(int dt, const void* q, int q_stride, void*
              "paged_attention: head size %d with group %d does not fit the local memory", d, group);
 #define AG_CASE(T, CHV)                                                                         \
   ag_launch<T, CHV>(q, q_stride, out, out_stride, kcache, vcache, block_table, table_stride,    \
-                    token_req, positions, n_tokens, nq, nkv, d, dv, P, window, scale, sink, score_bias, softcap, \
+                    token_req, positions, n_tokens, nq, nkv, d, dv, P, window, section, scale, sink, score_bias, softcap, \
                     bucket_of, far, rel, stream)
   if (dt == TK_F32) {
     if (ch == 64) AG_CASE(float, 64);

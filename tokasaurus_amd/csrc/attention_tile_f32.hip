@@ -4,7 +4,8 @@
 // window, key and value heads of different sizes, a scale of the model's choosing and a
 // learned sink per query head in the softmax's denominator; or, with `score_bias` (one number a
 // query head), no softmax at all: a visible key's weight is sigmoid(score + score_bias[head]), not
-// normalised over the keys (the sums of wavefronts and chunks are then added as they are).
+// normalised over the keys (the sums of wavefronts and chunks are then added as they are).  With `section` > 0 positions are
+// cut into sections at multiples of it, counted from a request's start, and a query sees only keys of its own section.
 //
 // A wavefront owns a tile of 16 "columns": tt = 16 / gg neighbouring tokens of one request
 // times gg neighbouring query heads of one kv head (gg = 1 for prompt portions; up to 16 for
@@ -99,7 +100,7 @@ __global__ __launch_bounds__(NW * TK_WAVE) void attention_tile_f32_kernel(
     const T* __restrict__ q, int q_stride, T* __restrict__ out, int out_stride, const T* __restrict__ kcache,
     const T* __restrict__ vcache, const int* __restrict__ block_table, int table_stride,
     const int* __restrict__ q_start, const int* __restrict__ kv_len, const int* __restrict__ tile_req,
-    const int* __restrict__ tile_row0, int nq, int nkv, int dk, int dv, int P, int window, float scale,
+    const int* __restrict__ tile_row0, int nq, int nkv, int dk, int dv, int P, int window, int section, float scale,
     const float* __restrict__ sink, const float* __restrict__ score_bias, int gg, AfterSum<T> after, ScoreShape shape,
     int chunk = 0, float* __restrict__ part = nullptr) {
   extern __shared__ float merge[];  // SPLIT: [waves][16] maxima, [waves][16] sums, [waves - 1][VT][4][64] weighted values
@@ -125,9 +126,11 @@ __global__ __launch_bounds__(NW * TK_WAVE) void attention_tile_f32_kernel(
   const int pos0 = kv - (q_end - row0);         // position of the tile's first token
   const int pos = pos0 + col / gg;              // of this column's token
   const int last_all = pos0 + n_tok - 1;  // the last key any column of the tile sees
-  // (PART) this workgroup's chunk: with a window the launch holds only as many chunks as a window touches, and
+  // (PART) this workgroup's chunk: with a window or sections the launch holds only as many chunks as those touch, and
   // blockIdx.z counts from the chunk of the first key that the tile sees (absolute multiples of `chunk` all the same)
-  const int first_seen = window > 0 ? max(0, pos0 - window + 1) : 0;
+  const int first_seen = section > 0 ? pos0 / section * section : (window > 0 ? max(0, pos0 - window + 1) : 0);
+  const int lo_col = section > 0 ? pos / section * section : 0;            // the first key of this column's section
+  const int lo_last = section > 0 ? last_all / section * section : 0;      // of the last column's
   const int zc = PART ? first_seen / chunk + (int)blockIdx.z : 0;
   const int last = PART ? min(last_all, (zc + 1) * chunk - 1) : last_all;  // the last this workgroup walks
   const int lo_tile = max(first_seen, PART ? zc * chunk : 0);
@@ -240,7 +243,7 @@ __global__ __launch_bounds__(NW * TK_WAVE) void attention_tile_f32_kernel(
     float sc[4];
     float tmax = -INFINITY;
     // a step that every column of the tile sees whole needs no masks (the same for all lanes)
-    const bool whole = k0 + 15 <= pos0 && (window <= 0 || last_all - k0 < window) && n_tok * gg == 16;
+    const bool whole = k0 + 15 <= pos0 && (window <= 0 || last_all - k0 < window) && k0 >= lo_last && n_tok * gg == 16;
     if (whole) {
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
@@ -252,7 +255,7 @@ __global__ __launch_bounds__(NW * TK_WAVE) void attention_tile_f32_kernel(
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
         const int kp = k0 + 4 * c + i;
-        const bool seen = live && kp <= pos && (window <= 0 || pos - kp < window);
+        const bool seen = live && kp <= pos && kp >= lo_col && (window <= 0 || pos - kp < window);
         sc[i] = seen ? (shaped ? shaped_score(shape, s[i] * scale, pos - kp, head, nq) : s[i] * scale) : -INFINITY;
         tmax = fmaxf(tmax, sc[i]);
       }
@@ -496,7 +499,7 @@ template <typename T, int KM, int VT>
 static void at_launch(dim3 grid, bool split, hipStream_t stream, const void* q, int q_stride, void* out, int out_stride,
                       const void* kcache, const void* vcache, const int* block_table, int table_stride,
                       const int* q_start, const int* kv_len, const int* tile_req, const int* tile_row0, int nq,
-                      int nkv, int dk, int dv, int P, int window, float scale, const float* sink, const float* score_bias,
+                      int nkv, int dk, int dv, int P, int window, int section, float scale, const float* sink, const float* score_bias,
                       int gg, int chunk, float* part, const float* vfreq, int v_pair_half, const void* gate, int gate_stride,
                       ScoreShape shape) {
   // halves of a head meet inside a lane only where the head fills the kernel's blocks of 16 (the entry point has checked)
@@ -507,7 +510,7 @@ static void at_launch(dim3 grid, bool split, hipStream_t stream, const void* q, 
     const size_t smem = sizeof(float) * (NW * 32 + (size_t)(NW - 1) * VT * 4 * TK_WAVE);
     hipLaunchKernelGGL((attention_tile_f32_kernel<T, KM, VT, true, NW, true>), grid, dim3(NW * TK_WAVE), smem, stream,
                        (const T*)q, q_stride, (T*)out, out_stride, (const T*)kcache, (const T*)vcache, block_table,
-                       table_stride, q_start, kv_len, tile_req, tile_row0, nq, nkv, dk, dv, P, window, scale, sink, score_bias, gg,
+                       table_stride, q_start, kv_len, tile_req, tile_row0, nq, nkv, dk, dv, P, window, section, scale, sink, score_bias, gg,
                        none, shape, chunk, part);
     hipLaunchKernelGGL((attention_tile_merge_kernel<T, VT>), dim3(grid.x, grid.y), dim3(VT * TK_WAVE), 0, stream, part, (int)grid.z,
                        (T*)out, out_stride, q_start, tile_req, tile_row0, nq, nkv, dv, sink, gg, score_bias ? 1 : 0, kv_len, after);
@@ -517,11 +520,11 @@ static void at_launch(dim3 grid, bool split, hipStream_t stream, const void* q, 
     const size_t smem = sizeof(float) * (NW * 32 + (size_t)(NW - 1) * VT * 4 * TK_WAVE);
     hipLaunchKernelGGL((attention_tile_f32_kernel<T, KM, VT, true, NW>), grid, dim3(NW * TK_WAVE), smem, stream,
                        (const T*)q, q_stride, (T*)out, out_stride, (const T*)kcache, (const T*)vcache, block_table,
-                       table_stride, q_start, kv_len, tile_req, tile_row0, nq, nkv, dk, dv, P, window, scale, sink, score_bias, gg, after, shape);
+                       table_stride, q_start, kv_len, tile_req, tile_row0, nq, nkv, dk, dv, P, window, section, scale, sink, score_bias, gg, after, shape);
   } else {
     hipLaunchKernelGGL((attention_tile_f32_kernel<T, KM, VT, false, AT_WAVES>), grid, dim3(AT_WAVES * TK_WAVE), 0, stream,
                        (const T*)q, q_stride, (T*)out, out_stride, (const T*)kcache, (const T*)vcache, block_table,
-                       table_stride, q_start, kv_len, tile_req, tile_row0, nq, nkv, dk, dv, P, window, scale, sink, score_bias, gg, after, shape);
+                       table_stride, q_start, kv_len, tile_req, tile_row0, nq, nkv, dk, dv, P, window, section, scale, sink, score_bias, gg, after, shape);
   }
 }
 
@@ -530,10 +533,11 @@ static void at_launch(dim3 grid, bool split, hipStream_t stream, const void* q, 
 TK_API int tk_attention_tile_f32(int dt, const void* q, int q_stride, void* out, int out_stride, const void* kcache,
                                  const void* vcache, const int* block_table, int table_stride, const int* q_start,
                                  const int* kv_len, const int* tile_req, const int* tile_row0, int n_tiles, int nq,
-                                 int nkv, int dk, int dv, int P, int window, float scale, const float* sink,
+                                 int nkv, int dk, int dv, int P, int window, int section, float scale, const float* sink,
                                  const float* score_bias, int gg, int split, int chunk, int chunks, float* part,
                                  const float* vfreq, int v_pair_half, const void* gate, int gate_stride, float softcap,
                                  const int* bucket_of, int far, const float* rel, hipStream_t stream) {
+  TK_REQUIRE(section <= 0 || window <= 0, "attention_tile_f32: a window or sections, not both");
   TK_REQUIRE(!rel || (bucket_of && far >= 0), "attention_tile_f32: a bias by distance needs its table of buckets");
   TK_REQUIRE(!(score_bias && (rel || softcap > 0.f)), "attention_tile_f32: sigmoid weights take neither a soft cap nor a bias by distance");
   const ScoreShape shape = {softcap, bucket_of, far, rel};
@@ -555,7 +559,7 @@ TK_API int tk_attention_tile_f32(int dt, const void* q, int q_stride, void* out,
   const dim3 grid(n_tiles, sp ? head_blocks : (head_blocks + AT_WAVES - 1) / AT_WAVES, parts ? chunks : 1);
   TK_REQUIRE(grid.y < 65536, "attention_tile_f32: too many heads");
 #define AT_ARGS grid, sp, stream, q, q_stride, out, out_stride, kcache, vcache, block_table, table_stride, q_start, kv_len, \
-                tile_req, tile_row0, nq, nkv, dk, dv, P, window, scale, sink, score_bias, gg, parts ? chunk : 0, part, vfreq, v_pair_half, \
+                tile_req, tile_row0, nq, nkv, dk, dv, P, window, section, scale, sink, score_bias, gg, parts ? chunk : 0, part, vfreq, v_pair_half, \
                 gate, gate_stride, shape
 #define AT_VT(T, KMV)                                      \
   do {                                                     \

@@ -88,6 +88,14 @@ __device__ __forceinline__ float silu_mul_bf16(float g, float u) {
   return s * ur;
 }
 
+// A gated activation with clamps, g sigmoid(alpha g) (u + 1) with g = min(gate, limit) and u = clamp(up, -limit, limit), as the
+// engine's storage type sees it: the operands rounded to it, 32-bit arithmetic, the result left for the caller to round.
+template <typename T>
+__device__ __forceinline__ float clamped_glu(float gate, float up, float limit, float alpha) {
+  const float g = fminf(round_to<T>(gate), limit), u = fminf(fmaxf(round_to<T>(up), -limit), limit);
+  return g / (1.0f + expf(-alpha * g)) * (u + 1.0f);
+}
+
 // Accesses that are coherent across the chip's dies (each has an L2 of its own): relaxed
 // atomics of agent scope, which the compiler turns into loads that go around, and stores that
 // write through, the caches.  Data that one workgroup of a running kernel writes and another

@@ -96,10 +96,7 @@ __device__ __forceinline__ void store4(const GemmArgs& a, f32x4_t v, f32x4_t up,
     if (EPI == EPI_SWIGLU) {
       const float g = v[j] * scale + bias_at(a, n + j, a.N), u = up[j] * scale + bias_at(a, a.N + n + j, 2 * a.N);
       if (a.glu_limit > 0.f) {
-        // (the operands rounded to the storage type first, as the separate kernel behind a product finds them)
-        const float gc = fminf(round_to<bf16_t>(g), a.glu_limit);
-        const float uc = fminf(fmaxf(round_to<bf16_t>(u), -a.glu_limit), a.glu_limit);
-        o[j] = gc / (1.0f + expf(-a.glu_alpha * gc)) * (uc + 1.0f);
+        o[j] = clamped_glu<bf16_t>(g, u, a.glu_limit, a.glu_alpha);
       } else if (a.glu_gelu) {
         const float gr = round_to<bf16_t>(g);
         o[j] = 0.5f * gr * (1.0f + tanhf(0.7978845608028654f * (gr + 0.044715f * gr * gr * gr))) * round_to<bf16_t>(u);

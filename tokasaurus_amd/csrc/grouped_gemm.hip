@@ -5,7 +5,7 @@
 //                         run of slots filled up to whole tiles of GG_TM or GS_M slots
 //   tk_grouped_gemm_bf16  C[c_row(slot), g * c_cols + n] = sum_k W[g][n][k] * A[a_row(slot), g * a_cols + k]
 //                         for the slots of every tile, g the tile's group; optionally the gated form
-//                         silu(gate) * up of two halves of W[g]
+//                         silu(gate) * up of two halves of W[g], or the gated form with clamps
 //   tk_expert_sum         per token the weighted sum of its pairs' rows, identity experts, shared expert
 //
 // A wavefront owns GG_TM = 64 slots x 64 outputs (32 in the gated form, for each of gate and up): weight rows
@@ -46,7 +46,11 @@ struct GroupedArgs {
   int N, K, slots;
   const float* row_scale;  // (gated form) a factor on a slot's sums of gate and up alike, row_scale[scale_row[slot]]; null: none
   const int* scale_row;
+  float limit, alpha;  // (gated form) limit > 0: the activation with clamps (clamped_glu of common.h) instead of silu
 };
+__device__ __forceinline__ float gg_gated(const GroupedArgs& a, float g, float u) {
+  return a.limit > 0.f ? clamped_glu<bf16_t>(g, u, a.limit, a.alpha) : silu_mul_bf16(g, u);
+}
 
 // NT: blocks of 16 outputs a wavefront; GLU: the gated form; F32: 32-bit output
 template <int NT, bool GLU, bool F32>
@@ -125,7 +129,7 @@ __global__ __launch_bounds__(GG_WAVES * TK_WAVE) void grouped_gemm_kernel(Groupe
       const int n = n0 + t * 16 + 4 * q;
       float y[4];
 #pragma unroll
-      for (int j = 0; j < 4; ++j) y[j] = GLU ? silu_mul_bf16(acc[t][mb][j] * f, acc[t + (GLU ? NT : 0)][mb][j] * f) : acc[t][mb][j];
+      for (int j = 0; j < 4; ++j) y[j] = GLU ? gg_gated(a, acc[t][mb][j] * f, acc[t + (GLU ? NT : 0)][mb][j] * f) : acc[t][mb][j];
       const size_t at = (size_t)crow * a.ldc + (size_t)g * a.c_cols + n;
 #pragma unroll
       for (int j = 0; j < 4; ++j) {
@@ -263,7 +267,7 @@ __global__ __launch_bounds__(256, 2) void grouped_gemm_staged_kernel(GroupedArgs
       const int n = n0 + (GLU ? wn * 32 + t * 16 : wn * 64 + t * 16) + 4 * q;
       float y[4];
 #pragma unroll
-      for (int j = 0; j < 4; ++j) y[j] = GLU ? silu_mul_bf16(acc[t][mb][j] * f, acc[t + (GLU ? 2 : 0)][mb][j] * f) : acc[t][mb][j];
+      for (int j = 0; j < 4; ++j) y[j] = GLU ? gg_gated(a, acc[t][mb][j] * f, acc[t + (GLU ? 2 : 0)][mb][j] * f) : acc[t][mb][j];
       if (n < a.N) gg_store4(dst + n, y, a.N - n);
     }
   }
@@ -272,7 +276,7 @@ __global__ __launch_bounds__(256, 2) void grouped_gemm_staged_kernel(GroupedArgs
 TK_API int tk_grouped_gemm_bf16(const void* A, int lda, const int* a_row, const int* c_row, const int* tile_group, int tiles,
                                 int groups_z, int a_cols, int c_cols, const void* W, size_t w_stride, void* C, int ldc,
                                 int N, int K, int slots, int glu, int out_f32, const float* row_scale, const int* scale_row,
-                                int tile_slots, hipStream_t stream) {
+                                int tile_slots, float limit, float alpha, hipStream_t stream) {
   TK_REQUIRE(A && W && C && N > 0 && K > 0 && slots >= 0 && tiles >= 0, "grouped_gemm: bad arguments");
   TK_REQUIRE(K % 8 == 0 && lda % 8 == 0 && a_cols % 8 == 0 && w_stride % 8 == 0 && (((uintptr_t)A | (uintptr_t)W) & 15) == 0,
              "grouped_gemm: rows of A and W must start at multiples of 16 bytes (K=%d lda=%d)", K, lda);
@@ -281,7 +285,7 @@ TK_API int tk_grouped_gemm_bf16(const void* A, int lda, const int* a_row, const 
   TK_REQUIRE(!(glu && out_f32), "grouped_gemm: the gated form writes the storage type");
   if (tiles == 0 || slots == 0) return 0;
   GroupedArgs a{(const bf16_t*)A, lda, a_row, c_row, tile_group, a_cols, c_cols, (const bf16_t*)W, w_stride, C, ldc, N, K, slots,
-                row_scale, scale_row};
+                row_scale, scale_row, limit, alpha};
   TK_REQUIRE(tile_slots == GG_TM || (tile_slots == GS_M && tile_group && !out_f32 && a_cols == 0 && c_cols == 0),
              "grouped_gemm: tiles of %d slots, or of %d with groups by tile and storage-type output", GG_TM, GS_M);
   if (tile_slots == GS_M) {
@@ -368,7 +372,7 @@ TK_API int tk_expert_sort(const int* ids, int pairs, int top, int experts, int m
 // --------------------------------------------------------------------------
 // out[t, c] = sum over the places k of token t, in order, of weights[t, k] * (y[t * top + k, c] for a routed expert,
 // h[t, c] for an identity expert), plus shared_gate[t] * shared[t, c].  y: [pairs, width] in the storage type.
-// `unit` != 0: a routed expert's row is added as it is.
+// `unit` != 0: a routed expert's row is added as it is.  weights null: equal parts, 1 / top each.
 // --------------------------------------------------------------------------
 __global__ __launch_bounds__(256) void expert_sum_kernel(const bf16_t* __restrict__ h, int h_stride, const bf16_t* __restrict__ y,
                                                          const int* __restrict__ ids, const float* __restrict__ weights,
@@ -381,7 +385,7 @@ __global__ __launch_bounds__(256) void expert_sum_kernel(const bf16_t* __restric
       const int e = ids[(size_t)t * top + k];
       if (e < 0) continue;
       const float v = e < experts ? __bfloat162float(y[((size_t)t * top + k) * width + c]) : __bfloat162float(h[(size_t)t * h_stride + c]);
-      acc = fmaf(unit && e < experts ? 1.f : weights[(size_t)t * top + k], v, acc);
+      acc = fmaf(unit && e < experts ? 1.f : (weights ? weights[(size_t)t * top + k] : 1.0f / (float)top), v, acc);
     }
     if (shared) acc = fmaf(shared_gate[t], shared[(size_t)t * width + c], acc);
     out[(size_t)t * width + c] = acc;
@@ -410,7 +414,7 @@ __global__ __launch_bounds__(256) void expert_sum_vec_kernel(const bf16_t* __res
         if (k0 + k >= top) continue;
         const int e = ids[t * top + k0 + k];
         if (e < 0) continue;
-        f[k] = unit && e < experts ? 1.f : weights[t * top + k0 + k];
+        f[k] = unit && e < experts ? 1.f : (weights ? weights[t * top + k0 + k] : 1.0f / (float)top);
         raw[k] = e < experts ? *(const uint4*)(y + (t * top + k0 + k) * width + c) : *(const uint4*)(h + t * h_stride + c);
       }
 #pragma unroll
@@ -432,7 +436,7 @@ __global__ __launch_bounds__(256) void expert_sum_vec_kernel(const bf16_t* __res
 
 TK_API int tk_expert_sum(const void* h, int h_stride, const void* y, const int* ids, const float* weights, const float* shared,
                          const float* shared_gate, float* out, int tokens, int width, int experts, int top, int unit, hipStream_t stream) {
-  TK_REQUIRE(h && y && ids && weights && out && (!shared || shared_gate) && tokens >= 0 && width > 0 && top > 0 && h_stride >= width,
+  TK_REQUIRE(h && y && ids && out && (!shared || shared_gate) && tokens >= 0 && width > 0 && top > 0 && h_stride >= width,
              "expert_sum: bad arguments");
   if (tokens == 0) return 0;
   if (width % 8 == 0 && h_stride % 8 == 0 && (((uintptr_t)h | (uintptr_t)y | (uintptr_t)out | (uintptr_t)shared) & 15) == 0) {

@@ -5,7 +5,8 @@
 //   tk_expert_route      per token: logits over all experts, their softmax or sigmoids, choice by score
 //                        (+ correction) inside the best groups of neighbouring experts, the chosen
 //                        experts' scores as weights; optionally the sigmoid gate of a shared expert
-//   tk_expert_gate_up    per (token, chosen expert): act(W_gate h) * (W_up h), of h or of weight * h
+//   tk_expert_lookup     the chosen experts from tables by token id, for all layers of a step at once
+//   tk_expert_gate_up    per (token, chosen expert): act(W_gate h) * (W_up h), of h or of weight * h, or the form with clamps
 //   tk_expert_combine    per token: sum of weight * W_down(...) over its experts, weight * h for an
 //                        identity expert, plus gate * (a shared expert's output)
 //   tk_head_linear       y[t, h, :] = W[h] x[t, h, :]: one matrix a head; optionally the leading part of a
@@ -207,16 +208,47 @@ TK_API int tk_expert_route(int dt, const void* h, int h_stride, const void* w_ro
 }
 
 // --------------------------------------------------------------------------
+// Experts by token id: for every layer with such a table, table[layer] [vocab][tops[layer]], the row of every token of the
+// step, ids[layer] [tokens][tops[layer]] (the layers' parts begin `at[layer]` * tokens numbers apart).  An id below 0 names
+// an entry of `last_token`, as in the embedding.  One launch a step for all layers: the choice rests on the ids alone.
+// --------------------------------------------------------------------------
+struct LookupLayer {
+  const int* table;
+  int top, at;
+};
+__global__ __launch_bounds__(256) void expert_lookup_kernel(const int* __restrict__ token_ids, const int* __restrict__ last_token, int vocab,
+                                                            const LookupLayer* __restrict__ layers, int* __restrict__ ids, int tokens) {
+  const int t = blockIdx.x * blockDim.x + threadIdx.x;
+  if (t >= tokens) return;
+  const LookupLayer l = layers[blockIdx.y];
+  int id = token_ids[t];
+  if (id < 0) id = last_token[-id - 1];
+  id = min(max(id, 0), vocab - 1);
+  for (int k = 0; k < l.top; ++k) ids[(size_t)l.at * tokens + (size_t)t * l.top + k] = l.table[(size_t)id * l.top + k];
+}
+
+TK_API int tk_expert_lookup(const int* token_ids, const int* last_token, int vocab, const void* layers, int* ids, int n_layers, int tokens,
+                            hipStream_t stream) {
+  TK_REQUIRE(token_ids && layers && ids && vocab > 0 && n_layers > 0 && n_layers < 65536 && tokens >= 0, "expert_lookup: bad arguments");
+  if (tokens == 0) return 0;
+  hipLaunchKernelGGL(expert_lookup_kernel, dim3((tokens + 255) / 256, n_layers), dim3(256), 0, stream, token_ids, last_token, vocab,
+                     (const LookupLayer*)layers, ids, tokens);
+  TK_CHECK_LAUNCH("expert_lookup");
+  return 0;
+}
+
+// --------------------------------------------------------------------------
 // inter[pair, j] = silu(W_gate[e] h)_j * (W_up[e] h)_j for pair = (token, place), e = ids[pair] a routed
 // expert (others are skipped).  w_gate_up: [experts][2 * ff][width], gate rows first.  `in_weights` (null or a number
 // a pair): the expert reads in_weights[pair] * h; the products being linear, the factor goes on their 32-bit sums.
+// `limit` > 0: the activation with clamps instead (clamped_glu of common.h).
 // Workgroup (pair, block of EX_ROWS outputs), a wavefront an output at a time.
 // --------------------------------------------------------------------------
 #define EX_ROWS 4  // one output a wavefront: a step of few tokens is a chain of loads, so many short workgroups
 template <typename T>
 __global__ __launch_bounds__(256) void expert_gate_up_kernel(
     const T* __restrict__ h, int h_stride, const T* __restrict__ w_gate_up, const int* __restrict__ ids,
-    const float* __restrict__ in_weights, T* __restrict__ inter, int width, int ff, int experts, int top) {
+    const float* __restrict__ in_weights, T* __restrict__ inter, int width, int ff, int experts, int top, float limit, float alpha) {
   const int pair = blockIdx.x;
   const int e = ids[pair];
   if (e < 0 || e >= experts) return;
@@ -233,6 +265,10 @@ __global__ __launch_bounds__(256) void expert_gate_up_kernel(
         g *= in_weights[pair];
         u *= in_weights[pair];
       }
+      if (limit > 0.f) {
+        inter[(size_t)pair * ff + j] = from_f32<T>(clamped_glu<T>(g, u, limit, alpha));
+        continue;
+      }
       // gate, up and the activation as the storage type sees them, as the dense feed-forward's epilogue
       const float gr = round_to<T>(g), ur = round_to<T>(u);
       const float a = round_to<T>(gr / (1.0f + expf(-gr)));
@@ -242,7 +278,7 @@ __global__ __launch_bounds__(256) void expert_gate_up_kernel(
 }
 
 TK_API int tk_expert_gate_up(int dt, const void* h, int h_stride, const void* w_gate_up, const int* ids, const float* in_weights, void* inter,
-                             int tokens, int width, int ff, int experts, int top, hipStream_t stream) {
+                             int tokens, int width, int ff, int experts, int top, float limit, float alpha, hipStream_t stream) {
   TK_REQUIRE(tokens >= 0 && width > 0 && ff > 0 && experts > 0 && top > 0 && h_stride >= width,
              "expert_gate_up: bad sizes tokens=%d width=%d ff=%d experts=%d top=%d", tokens, width, ff, experts, top);
   TK_REQUIRE(h && w_gate_up && ids && inter, "expert_gate_up: a pointer is missing");
@@ -251,10 +287,10 @@ TK_API int tk_expert_gate_up(int dt, const void* h, int h_stride, const void* w_
   TK_REQUIRE(grid.y < 65536, "expert_gate_up: an expert of %d rows is too large", ff);
   if (dt == TK_F32)
     hipLaunchKernelGGL(expert_gate_up_kernel<float>, grid, dim3(256), 0, stream, (const float*)h, h_stride,
-                       (const float*)w_gate_up, ids, in_weights, (float*)inter, width, ff, experts, top);
+                       (const float*)w_gate_up, ids, in_weights, (float*)inter, width, ff, experts, top, limit, alpha);
   else
     hipLaunchKernelGGL(expert_gate_up_kernel<bf16_t>, grid, dim3(256), 0, stream, (const bf16_t*)h, h_stride,
-                       (const bf16_t*)w_gate_up, ids, in_weights, (bf16_t*)inter, width, ff, experts, top);
+                       (const bf16_t*)w_gate_up, ids, in_weights, (bf16_t*)inter, width, ff, experts, top, limit, alpha);
   TK_CHECK_LAUNCH("expert_gate_up");
   return 0;
 }
@@ -264,7 +300,7 @@ TK_API int tk_expert_gate_up(int dt, const void* h, int h_stride, const void* w_
 //     weights[t, k] * (W_down[e] inter[t, k])_c       e = ids[t, k] a routed expert
 //     weights[t, k] * h[t, c]                         e an identity expert (e >= experts)
 // plus shared_gate[t] * shared[t, c] when a shared expert's output is given.  out is 32-bit.  `unit` != 0: a routed
-// expert's output is added as it is (its weight went on what it read).
+// expert's output is added as it is (its weight went on what it read).  weights null: equal parts, 1 / top each.
 // w_down: [experts][width][ff].  Workgroup (token, block of EX_ROWS columns).
 // --------------------------------------------------------------------------
 template <typename T>
@@ -280,7 +316,7 @@ __global__ __launch_bounds__(256) void expert_combine_kernel(
     for (int k = 0; k < top; ++k) {
       const int e = ids[(size_t)t * top + k];
       if (e < 0) continue;
-      const float g = unit && e < experts ? 1.f : weights[(size_t)t * top + k];
+      const float g = unit && e < experts ? 1.f : (weights ? weights[(size_t)t * top + k] : 1.0f / (float)top);
       float y;
       if (e < experts)
         y = round_to<T>(wave_dot<T>(w_down + ((size_t)e * width + c) * ff, inter + ((size_t)t * top + k) * ff, ff));
@@ -298,7 +334,7 @@ TK_API int tk_expert_combine(int dt, const void* h, int h_stride, const void* in
                              int width, int ff, int experts, int top, int unit, hipStream_t stream) {
   TK_REQUIRE(tokens >= 0 && width > 0 && ff > 0 && experts > 0 && top > 0 && h_stride >= width,
              "expert_combine: bad sizes tokens=%d width=%d ff=%d experts=%d top=%d", tokens, width, ff, experts, top);
-  TK_REQUIRE(h && inter && w_down && ids && weights && out && (!shared || shared_gate), "expert_combine: a pointer is missing");
+  TK_REQUIRE(h && inter && w_down && ids && out && (!shared || shared_gate), "expert_combine: a pointer is missing");
   if (tokens == 0) return 0;
   const dim3 grid(tokens, (width + EX_ROWS - 1) / EX_ROWS);
   TK_REQUIRE(grid.y < 65536, "expert_combine: a width of %d is too large", width);

@@ -447,27 +447,59 @@ TK_API int tk_residual_norm(int dt, const float* x, const float* a, const float*
 // The update of a stream whose branches are normed before they are added (a norm in front of and
 // behind every sublayer), one row a workgroup:
 //     x_out = x + a / sqrt(mean(a^2) + eps_b) * wb
+// or, PAIR (a sublayer made of two side by side, each with a norm of its own behind it; x may then be null for zeros),
+//     x_out = x + mult * (a / sqrt(mean(a^2) + eps_b) * wb + a2 / sqrt(mean(a2^2) + eps_b) * wb2)
 // and, when w is given, the row of the norm that reads the new stream,
 //     h = x_out / sqrt(mean(x_out^2) + eps) * w     rounded once to T;
 // with h and no w, h is x_out itself rounded once to T (for sublayers that read the stream unnormed).
-// x, a, wb, w are 32-bit.  x_out may be x itself.  The row is held in registers between the
+// x, a, a2, wb, wb2, w are 32-bit.  x_out may be x itself.  The row is held in registers between the
 // passes when the width allows (multiples of 4 up to 4 * 256 * RN_QUADS), else read back.
 // --------------------------------------------------------------------------
-template <typename T>
+struct PostNormPair {  // the second branch (PAIR)
+  const float *a, *w;
+  float mult;
+};
+// both branches' sums of squares over a workgroup, with the barriers of one
+__device__ __forceinline__ void block_sum2(float& u, float& v, float* scratch) {
+  const int lane = threadIdx.x & (TK_WAVE - 1), wave = threadIdx.x / TK_WAVE, nwaves = blockDim.x / TK_WAVE;
+  u = wave_sum(u);
+  v = wave_sum(v);
+  __syncthreads();
+  if (lane == 0) {
+    scratch[wave] = u;
+    scratch[8 + wave] = v;
+  }
+  __syncthreads();
+  u = v = 0.f;
+  for (int w = 0; w < nwaves; ++w) {
+    u += scratch[w];
+    v += scratch[8 + w];
+  }
+}
+
+template <typename T, bool PAIR>
 __global__ __launch_bounds__(256) void post_norm_residual_kernel(
-    const float* x, const float* __restrict__ a, const float* __restrict__ wb, float eps_b,
+    const float* x, const float* __restrict__ a, const float* __restrict__ wb, float eps_b, PostNormPair p,
     float* x_out, const float* __restrict__ w, float eps, T* __restrict__ h, int hidden) {
   __shared__ float red[16];
   const size_t row = (size_t)blockIdx.x * hidden;
-  float sa = 0.f;
+  float sa = 0.f, sp = 0.f;
   for (int i = threadIdx.x; i < hidden; i += blockDim.x) {
     const float y = a[row + i];
     sa = fmaf(y, y, sa);
+    if (PAIR) {
+      const float z = p.a[row + i];
+      sp = fmaf(z, z, sp);
+    }
   }
-  const float rb = 1.0f / sqrtf(block_sum(sa, red) / (float)hidden + eps_b);
+  if (PAIR) block_sum2(sa, sp, red);
+  else sa = block_sum(sa, red);
+  const float rb = 1.0f / sqrtf(sa / (float)hidden + eps_b), rp = PAIR ? 1.0f / sqrtf(sp / (float)hidden + eps_b) : 0.f;
   float ss = 0.f;
   for (int i = threadIdx.x; i < hidden; i += blockDim.x) {
-    const float v = x[row + i] + a[row + i] * rb * wb[i];
+    float v;
+    if (PAIR) v = fmaf(p.mult, a[row + i] * rb * wb[i] + p.a[row + i] * rp * p.w[i], x ? x[row + i] : 0.f);
+    else v = x[row + i] + a[row + i] * rb * wb[i];
     x_out[row + i] = v;
     ss = fmaf(v, v, ss);
   }
@@ -481,15 +513,15 @@ __global__ __launch_bounds__(256) void post_norm_residual_kernel(
     h[row + i] = from_f32<T>(x_out[row + i] * rstd * w[i]);
 }
 
-template <typename T>
+template <typename T, bool PAIR>
 __global__ __launch_bounds__(256) void post_norm_residual_vec_kernel(
-    const float* x, const float* __restrict__ a, const float* __restrict__ wb, float eps_b,
+    const float* x, const float* __restrict__ a, const float* __restrict__ wb, float eps_b, PostNormPair p,
     float* x_out, const float* __restrict__ w, float eps, T* __restrict__ h, int hidden) {
   __shared__ float red[16];
   const size_t row = (size_t)blockIdx.x * hidden;
   const int quads = hidden / 4;
-  float4 v[RN_QUADS];
-  float sa = 0.f;
+  float4 v[RN_QUADS], z[PAIR ? RN_QUADS : 1];
+  float sa = 0.f, sp = 0.f;
 #pragma unroll
   for (int j = 0; j < RN_QUADS; ++j) {
     const int i = threadIdx.x + j * 256;
@@ -497,18 +529,33 @@ __global__ __launch_bounds__(256) void post_norm_residual_vec_kernel(
       v[j] = ((const float4*)(a + row))[i];
       sa = fmaf(v[j].x, v[j].x, sa); sa = fmaf(v[j].y, v[j].y, sa);
       sa = fmaf(v[j].z, v[j].z, sa); sa = fmaf(v[j].w, v[j].w, sa);
+      if constexpr (PAIR) {
+        z[j] = ((const float4*)(p.a + row))[i];
+        sp = fmaf(z[j].x, z[j].x, sp); sp = fmaf(z[j].y, z[j].y, sp);
+        sp = fmaf(z[j].z, z[j].z, sp); sp = fmaf(z[j].w, z[j].w, sp);
+      }
     }
   }
-  const float rb = 1.0f / sqrtf(block_sum(sa, red) / (float)hidden + eps_b);
+  if (PAIR) block_sum2(sa, sp, red);
+  else sa = block_sum(sa, red);
+  const float rb = 1.0f / sqrtf(sa / (float)hidden + eps_b), rp = PAIR ? 1.0f / sqrtf(sp / (float)hidden + eps_b) : 0.f;
   float ss = 0.f;
 #pragma unroll
   for (int j = 0; j < RN_QUADS; ++j) {
     const int i = threadIdx.x + j * 256;
     if (i < quads) {
-      const float4 xv = ((const float4*)(x + row))[i];
+      const float4 xv = !PAIR || x ? ((const float4*)(x + row))[i] : make_float4(0.f, 0.f, 0.f, 0.f);
       const float4 g = ((const float4*)wb)[i];
-      v[j].x = xv.x + v[j].x * rb * g.x; v[j].y = xv.y + v[j].y * rb * g.y;
-      v[j].z = xv.z + v[j].z * rb * g.z; v[j].w = xv.w + v[j].w * rb * g.w;
+      if constexpr (PAIR) {
+        const float4 k = ((const float4*)p.w)[i];
+        v[j].x = fmaf(p.mult, v[j].x * rb * g.x + z[j].x * rp * k.x, xv.x);
+        v[j].y = fmaf(p.mult, v[j].y * rb * g.y + z[j].y * rp * k.y, xv.y);
+        v[j].z = fmaf(p.mult, v[j].z * rb * g.z + z[j].z * rp * k.z, xv.z);
+        v[j].w = fmaf(p.mult, v[j].w * rb * g.w + z[j].w * rp * k.w, xv.w);
+      } else {
+        v[j].x = xv.x + v[j].x * rb * g.x; v[j].y = xv.y + v[j].y * rb * g.y;
+        v[j].z = xv.z + v[j].z * rb * g.z; v[j].w = xv.w + v[j].w * rb * g.w;
+      }
       ((float4*)(x_out + row))[i] = v[j];
       ss = fmaf(v[j].x, v[j].x, ss); ss = fmaf(v[j].y, v[j].y, ss);
       ss = fmaf(v[j].z, v[j].z, ss); ss = fmaf(v[j].w, v[j].w, ss);
@@ -528,21 +575,29 @@ __global__ __launch_bounds__(256) void post_norm_residual_vec_kernel(
   }
 }
 
-TK_API int tk_post_norm_residual(int dt, const float* x, const float* a, const float* wb, float eps_b, float* x_out,
-                                 const float* w, float eps, void* h, int rows, int hidden, hipStream_t stream) {
+// a2 (null without a second branch), wb2, mult: see above
+TK_API int tk_post_norm_residual(int dt, const float* x, const float* a, const float* wb, float eps_b, const float* a2, const float* wb2,
+                                 float mult, float* x_out, const float* w, float eps, void* h, int rows, int hidden, hipStream_t stream) {
   TK_REQUIRE(rows >= 0 && hidden > 0, "post_norm_residual: bad sizes %d %d", rows, hidden);
-  TK_REQUIRE(x && a && wb && x_out && (!w || h), "post_norm_residual: a pointer is missing");
+  TK_REQUIRE((x || a2) && a && wb && x_out && (!w || h) && (!a2 || wb2), "post_norm_residual: a pointer is missing");
   TK_REQUIRE(w || !h || dt != TK_F32, "post_norm_residual: 32-bit rows of the stream itself are the stream");
+  TK_REQUIRE(a2 || mult == 1.f, "post_norm_residual: a factor goes with a second branch");
   if (rows == 0) return 0;
-  const uintptr_t all = (uintptr_t)x | (uintptr_t)a | (uintptr_t)wb | (uintptr_t)x_out | (uintptr_t)w;
+  const PostNormPair p{a2, wb2, mult};
+  const uintptr_t all = (uintptr_t)x | (uintptr_t)a | (uintptr_t)wb | (uintptr_t)x_out | (uintptr_t)w | (uintptr_t)a2 | (uintptr_t)wb2;
   const bool vec = hidden % 4 == 0 && hidden <= 4 * 256 * RN_QUADS && (all & 15) == 0;
-#define PNR_LAUNCH(K, T) hipLaunchKernelGGL(K<T>, dim3(rows), dim3(256), 0, stream, x, a, wb, eps_b, x_out, w, eps, (T*)h, hidden)
-  if (vec) {
-    if (dt == TK_F32) PNR_LAUNCH(post_norm_residual_vec_kernel, float); else PNR_LAUNCH(post_norm_residual_vec_kernel, bf16_t);
-  } else {
-    if (dt == TK_F32) PNR_LAUNCH(post_norm_residual_kernel, float); else PNR_LAUNCH(post_norm_residual_kernel, bf16_t);
-  }
-#undef PNR_LAUNCH
+#define PNR_ARGS(T) dim3(rows), dim3(256), 0, stream, x, a, wb, eps_b, p, x_out, w, eps, (T*)h, hidden
+#define PNR_CASE(T)                                                                                              \
+  do {                                                                                                           \
+    if (vec && a2) hipLaunchKernelGGL((post_norm_residual_vec_kernel<T, true>), PNR_ARGS(T));           \
+    else if (vec) hipLaunchKernelGGL((post_norm_residual_vec_kernel<T, false>), PNR_ARGS(T));           \
+    else if (a2) hipLaunchKernelGGL((post_norm_residual_kernel<T, true>), PNR_ARGS(T));                           \
+    else hipLaunchKernelGGL((post_norm_residual_kernel<T, false>), PNR_ARGS(T));                                  \
+  } while (0)
+  if (dt == TK_F32) PNR_CASE(float);
+  else PNR_CASE(bf16_t);
+#undef PNR_CASE
+#undef PNR_ARGS
   TK_CHECK_LAUNCH("post_norm_residual");
   return 0;
 }

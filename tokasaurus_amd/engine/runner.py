@@ -378,7 +378,7 @@ class ModelRunner:
         if len(pages) != len(self.groups):
             raise ValueError(f"{len(pages)} page counts for {len(self.groups)} cache groups")
         # a request's length is bounded by the pools that keep every key; a windowed group recycles its pages
-        whole = [n for n, g in zip(pages, self.groups) if not g.need.window] or pages
+        whole = [n for n, g in zip(pages, self.groups) if g.need.keeps_all] or pages
         limit = min([self.max_positions] + [n * page_size for n in whole])
         if max_tokens_per_request is not None:
             limit = min(limit, max_tokens_per_request)

@@ -34,15 +34,16 @@ _SIGNATURES: dict[str, dict[str, list]] = {
         "tk_add_bias": [c_int, _P, _P, c_int, c_int, _P],
         "tk_head_rmsnorm": [c_int, _P, c_int, _P, c_int, c_int, c_int, c_int, c_int, c_float, _P],
         "tk_paged_attention_generic": [c_int, _P, c_int, _P, c_int, _P, _P, _P, c_int, _P, _P]
-        + [c_int] * 7
+        + [c_int] * 8
         + [c_float, _P, _P, c_float, _P, c_int, _P, _P],
         "tk_paged_attention_generic_fits": [c_int, c_int, c_int, c_int],
         "tk_add": [c_int, _P, _P, _P, c_size_t, _P],
         "tk_embed_scaled": [c_int, _P, _P, _P, _P, c_int, c_int, c_int, c_float, _P, _P, c_int, _P],
         "tk_depth_average": [c_int, _P, c_size_t, c_int, _P, _P, _P, _P, _P, c_float, c_float, _P, c_int, c_int, _P, _P, c_float, _P],
-        "tk_linear_attention": [c_int, _P, c_int, c_int, c_int, c_int, _P, _P, _P, _P, c_size_t, _P, _P, _P, _P] + [c_int] * 6 + [_P],
-        "tk_linear_attention_rec_width": [c_int, c_int, c_int],
-        "tk_group_norm_gate": [c_int, _P, _P, c_int, _P, c_float, c_float, _P, c_int, c_int, c_int, c_int, _P],
+        "tk_linear_attention": [c_int, _P, _P],
+        "tk_linear_attention_state_words": [c_int] * 4,
+        "tk_linear_attention_work_words": [c_int] * 5,
+        "tk_group_norm_gate": [c_int, _P, c_int, _P, c_int, c_int, _P, c_int, _P, c_float, c_float, _P, c_int, c_int, c_int, c_int, _P],
         "tk_sigmoid_gate": [c_int, _P, c_int, _P, c_int, c_float, _P, c_int, c_int, c_int, _P],
         "tk_short_conv": [c_int, _P, c_int, _P, c_int, _P, c_size_t, _P, _P, _P, _P] + [c_int] * 4 + [_P],
         "tk_gelu_glu": [c_int, _P, _P, c_int, c_int, _P],
@@ -60,14 +61,15 @@ _SIGNATURES: dict[str, dict[str, list]] = {
         "tk_scale_values": [_P, c_size_t, c_float, _P],
         "tk_clamped_glu": [c_int, _P, _P, c_int, c_int, c_float, c_float, _P],
         "tk_gather_keys": [c_int, _P, _P, c_int, _P, _P, _P] + [c_int] * 5 + [_P],
-        "tk_post_norm_residual": [c_int, _P, _P, _P, c_float, _P, _P, c_float, _P, c_int, c_int, _P],
+        "tk_post_norm_residual": [c_int, _P, _P, _P, c_float, _P, _P, c_float, _P, _P, c_float, _P, c_int, c_int, _P],
         "tk_concat_cast": [c_int, _P, _P, _P, c_int, c_int, _P],
         "tk_expert_route": [c_int, _P, c_int, _P, _P, _P] + [c_int] * 6 + [_P, _P, _P, c_float, c_int, _P],
-        "tk_expert_gate_up": [c_int, _P, c_int, _P, _P, _P, _P] + [c_int] * 5 + [_P],
+        "tk_expert_gate_up": [c_int, _P, c_int, _P, _P, _P, _P] + [c_int] * 5 + [c_float, c_float, _P],
+        "tk_expert_lookup": [_P, _P, c_int, _P, _P, c_int, c_int, _P],
         "tk_expert_combine": [c_int, _P, c_int, _P, _P, _P, _P, _P, _P, _P] + [c_int] * 6 + [_P],
         "tk_head_linear": [c_int, _P, c_int, _P, _P, c_int, c_int] + [c_int] * 4 + [_P, _P, c_int, c_int, c_float, _P, c_int, _P],
         "tk_squared_relu": [c_int, _P, c_size_t, _P],
-        "tk_attention_tile_f32": [c_int, _P, c_int, _P, c_int, _P, _P, _P, c_int, _P, _P, _P, _P] + [c_int] * 7
+        "tk_attention_tile_f32": [c_int, _P, c_int, _P, c_int, _P, _P, _P, c_int, _P, _P, _P, _P] + [c_int] * 8
         + [c_float, _P, _P, c_int, c_int, c_int, c_int, _P, _P, c_int, _P, c_int, c_float, _P, c_int, _P, _P],
         "tk_attention_tile_turns_halves": [c_int],
         "tk_attention_tile_part_words": [c_int],
@@ -90,7 +92,7 @@ _SIGNATURES: dict[str, dict[str, list]] = {
         "tk_gemm_skinny_bf16": [_P, c_int, _P, _P, c_int, _P, c_int, _P] + [c_int] * 9 + [_P],
         "tk_gemm_skinny_parts": [c_int, c_int, c_int],
         "tk_grouped_gemm_bf16": [_P, c_int, _P, _P, _P, c_int, c_int, c_int, c_int, _P, c_size_t, _P, c_int, c_int, c_int, c_int,
-                                 c_int, c_int, _P, _P, c_int, _P],
+                                 c_int, c_int, _P, _P, c_int, c_float, c_float, _P],
         "tk_expert_sort": [_P, c_int, c_int, c_int, c_int, c_int, _P, _P, _P, _P],
         "tk_expert_sum": [_P, c_int, _P, _P, _P, _P, _P, _P, c_int, c_int, c_int, c_int, c_int, _P],
     },

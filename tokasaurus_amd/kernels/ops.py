@@ -358,6 +358,7 @@ def paged_attention_generic(
     score_bias: torch.Tensor | None = None,
     softcap: float = 0.0,
     distance_bias: "DistanceBias | None" = None,
+    section: int = 0,
 ) -> torch.Tensor:
     """Attention of every token over its request's pages (see rope_append for
     the page layout).  ``q`` is 2-d, its first nq*d columns are the query heads.
@@ -366,7 +367,8 @@ def paged_attention_generic(
     softmax's denominator once, with no key and no value.  ``score_bias`` (32-bit, one number a
     query head): no softmax; a visible key's weight is sigmoid(score + score_bias[head]), not normalised.
     ``softcap`` (> 0): a scaled score becomes softcap * tanh(score / softcap).  ``distance_bias``: a learned
-    number by (bucket of the distance, head) is added to the score after that."""
+    number by (bucket of the distance, head) is added to the score after that.  ``section`` (> 0, without a window): positions
+    are cut at multiples of it and a query sees only keys of its own section."""
     _gpu(q, kcache, vcache, block_table, token_req, positions, sink, score_bias)
     db = _checked_distance_bias(distance_bias, nq)
     vd = head_dim if value_dim is None else int(value_dim)
@@ -403,6 +405,7 @@ def paged_attention_generic(
         vd,
         page_size,
         int(window),
+        int(section),
         float(scale if scale is not None else 1.0 / math.sqrt(head_dim)),
         sink.data_ptr() if sink is not None else None,
         score_bias.data_ptr() if score_bias is not None else None,
@@ -1229,6 +1232,64 @@ def depth_average(hist: torch.Tensor, count: int, weights: torch.Tensor, last: t
 # linear attention with a decay, and what stands around it
 # --------------------------------------------------------------------------
 
+class _LinearAttentionArgs(ctypes.Structure):
+    """The arguments of tk_linear_attention (struct LaArgs of linear_attention.hip)."""
+
+    _fields_ = [
+        ("proj", ctypes.c_void_p), ("ld", ctypes.c_int), ("q_off", ctypes.c_int), ("k_off", ctypes.c_int), ("v_off", ctypes.c_int),
+        ("decay", ctypes.c_void_p), ("forget_bias", ctypes.c_void_p), ("forget_low", ctypes.c_void_p),
+        ("low_off", ctypes.c_int), ("rank", ctypes.c_int), ("low_up", ctypes.c_void_p), ("low_bias", ctypes.c_void_p), ("tau", ctypes.c_float),
+        ("i_off", ctypes.c_int), ("f_off", ctypes.c_int), ("i_bias", ctypes.c_void_p), ("f_bias", ctypes.c_void_p),
+        ("cap", ctypes.c_float), ("q_scale", ctypes.c_float), ("state", ctypes.c_void_p), ("state_stride", ctypes.c_size_t),
+        ("q_start", ctypes.c_void_p), ("slots", ctypes.c_void_p), ("positions", ctypes.c_void_p), ("rec", ctypes.c_void_p),
+        ("o", ctypes.c_void_p), ("floor", ctypes.c_void_p), ("o_head", ctypes.c_int), ("n_tokens", ctypes.c_int),
+        ("n_requests", ctypes.c_int), ("H", ctypes.c_int), ("dk", ctypes.c_int), ("dv", ctypes.c_int), ("longest", ctypes.c_int),
+    ]
+
+
+LA_CONSTANT, LA_FORGET, LA_CHANNEL, LA_MEMORY = range(4)  # the forms of tk_linear_attention
+
+
+def linear_attention_state_words(heads: int, key_dim: int, value_dim: int, memory: bool = False) -> int:
+    """32-bit numbers a request keeps for a linear-attention mixer (``memory``: of ``matrix_memory``'s form)."""
+    if memory:  # a column more for the keys' sum, and two rows of running maxima
+        return -(-(heads * (value_dim + 1) * key_dim + 2 * heads) // 4) * 4
+    return heads * value_dim * key_dim
+
+
+def _linear_attention(mode: int, proj: torch.Tensor, q_off: int, k_off: int, v_off: int, state: torch.Tensor, q_start: torch.Tensor,
+                      slots: torch.Tensor, heads: int, key_dim: int, value_dim: int, longest: int | None, extra: dict,
+                      o_head: int | None = None) -> torch.Tensor:
+    """What the forms of the recurrence share: checks, working memory, the result [tokens, heads * o_head]."""
+    _gpu(proj, state, q_start, slots)
+    _need(proj.dim() == 2 and proj.dtype == torch.float32 and proj.stride(1) == 1, "linear_attention: 32-bit rows with unit inner stride")
+    H, dk, dv = int(heads), int(key_dim), int(value_dim)
+    n, width = proj.shape
+    for off, size in ((q_off, H * dk), (k_off, H * dk), (v_off, H * dv)):
+        _need(0 <= off and off + size <= width, "linear_attention: a part lies outside the rows")
+    words = linear_attention_state_words(H, dk, dv, mode == LA_MEMORY)
+    _need(state.dim() == 2 and state.dtype == torch.float32 and state.is_contiguous() and state.shape[1] >= words,
+          f"linear_attention: the state must be contiguous float32 [slots, {words}]")
+    _i32(q_start, "q_start")
+    _i32(slots, "slots")
+    _need(q_start.numel() == slots.numel() + 1, "linear_attention: one slot a request")
+    _need(dk <= 512, f"linear_attention: heads of up to 512 key channels, not {dk}")
+    o_head = dv if o_head is None else o_head
+    o = torch.empty((n, H * o_head), dtype=torch.float32, device=proj.device)
+    if n:
+        longest = max(1, int(n if longest is None else longest))
+        # the activated rows that the recurrence reads: passes over the step's tokens in front of it (a step of single
+        # tokens computes them in the recurrence's own kernel)
+        work = load("core").tk_linear_attention_work_words(mode, H, dk, dv, longest)
+        rec = torch.empty((n, work), dtype=torch.float32, device=proj.device) if work else None
+        a = _LinearAttentionArgs(proj=proj.data_ptr(), ld=proj.stride(0), q_off=int(q_off), k_off=int(k_off), v_off=int(v_off),
+                                 state=state.data_ptr(), state_stride=state.stride(0), q_start=q_start.data_ptr(), slots=slots.data_ptr(),
+                                 rec=rec.data_ptr() if rec is not None else None, o=o.data_ptr(), o_head=o_head, n_tokens=n,
+                                 n_requests=slots.numel(), H=H, dk=dk, dv=dv, longest=longest, **extra)
+        call("tk_linear_attention", mode, ctypes.addressof(a), _stream())
+    return o
+
+
 def linear_attention(proj: torch.Tensor, q_off: int, k_off: int, v_off: int, state: torch.Tensor, q_start: torch.Tensor,
                      slots: torch.Tensor, heads: int, key_dim: int, value_dim: int, decay: torch.Tensor | None = None,
                      forget_bias: torch.Tensor | None = None, forget_low: torch.Tensor | None = None,
@@ -1241,59 +1302,89 @@ def linear_attention(proj: torch.Tensor, q_off: int, k_off: int, v_off: int, sta
     it is.  ``state`` [slots + 1, heads * value_dim * key_dim] (32-bit) is read and written in the requests'
     ``slots``.  ``longest``: the most tokens a request brings in this step (the launch's form depends on it, the sums
     do not; by default the step's tokens).  Returns o [tokens, heads * value_dim] in 32-bit."""
-    _gpu(proj, state, q_start, slots, decay, forget_bias, forget_low)
-    _need(proj.dim() == 2 and proj.dtype == torch.float32 and proj.stride(1) == 1, "linear_attention: 32-bit rows with unit inner stride")
-    H, dk, dv = int(heads), int(key_dim), int(value_dim)
-    n, width = proj.shape
-    for off, size in ((q_off, H * dk), (k_off, H * dk), (v_off, H * dv)):
-        _need(0 <= off and off + size <= width, "linear_attention: a part lies outside the rows")
-    _need(state.dim() == 2 and state.dtype == torch.float32 and state.is_contiguous() and state.shape[1] >= H * dk * dv,
-          "linear_attention: the state must be contiguous float32 [slots, heads * dv * dk]")
-    _i32(q_start, "q_start")
-    _i32(slots, "slots")
-    _need(q_start.numel() == slots.numel() + 1, "linear_attention: one slot a request")
+    _gpu(decay, forget_bias, forget_low)
     constant = decay is not None
     _need(constant != (forget_bias is not None and forget_low is not None), "linear_attention: a decay a head, or a forget gate's bias and bound")
-    _f32_vector(decay, H, "linear_attention: the decays")
-    _f32_vector(forget_bias, H * dk, "linear_attention: the forget gate's bias")
-    _f32_vector(forget_low, H * dk, "linear_attention: the forget gate's lower bound")
-    _need(dk <= 512, f"linear_attention: heads of up to 512 key channels, not {dk}")
-    o = torch.empty((n, H * dv), dtype=torch.float32, device=proj.device)
-    if n:
-        longest = max(1, int(n if longest is None else longest))
-        # the activated rows that the recurrence reads: one pass over the step's tokens in front of it (a step of single
-        # tokens computes them in the recurrence's own kernel)
-        rec = (torch.empty((n, load("core").tk_linear_attention_rec_width(H, dk, dv)), dtype=torch.float32, device=proj.device)
-               if longest > 1 else None)
-        call("tk_linear_attention", 0 if constant else 1, proj.data_ptr(), proj.stride(0), int(q_off), int(k_off), int(v_off),
-             decay.data_ptr() if constant else None, forget_bias.data_ptr() if not constant else None,
-             forget_low.data_ptr() if not constant else None, state.data_ptr(), state.stride(0), q_start.data_ptr(),
-             slots.data_ptr(), rec.data_ptr() if rec is not None else None, o.data_ptr(), n, slots.numel(), H, dk, dv, longest,
-             _stream())
-    return o
+    _f32_vector(decay, heads, "linear_attention: the decays")
+    _f32_vector(forget_bias, heads * key_dim, "linear_attention: the forget gate's bias")
+    _f32_vector(forget_low, heads * key_dim, "linear_attention: the forget gate's lower bound")
+    extra = dict(decay=decay.data_ptr()) if constant else dict(forget_bias=forget_bias.data_ptr(), forget_low=forget_low.data_ptr())
+    return _linear_attention(LA_CONSTANT if constant else LA_FORGET, proj, q_off, k_off, v_off, state, q_start, slots, heads, key_dim,
+                             value_dim, longest, extra)
+
+
+def gated_linear_attention(proj: torch.Tensor, q_off: int, k_off: int, v_off: int, low_off: int, low_up: torch.Tensor,
+                           low_bias: torch.Tensor, tau: float, q_scale: float, state: torch.Tensor, q_start: torch.Tensor,
+                           slots: torch.Tensor, heads: int, key_dim: int, value_dim: int, longest: int | None = None) -> torch.Tensor:
+    """The recurrence of ``linear_attention`` with q (times ``q_scale``), k and v as they are and a decay per head and key
+    channel, ``a = sigmoid(z)^(1 / tau)`` with ``z = low_up^T low + low_bias``: ``low`` are the sums from column ``low_off``
+    on, ``low_up`` [rank, heads * key_dim] and ``low_bias`` are 32-bit."""
+    _gpu(low_up, low_bias)
+    _need(low_up.dim() == 2 and low_up.shape[1] == heads * key_dim and low_up.dtype == torch.float32 and low_up.is_contiguous(),
+          "gated_linear_attention: the low-rank projection's second matrix must be contiguous float32 [rank, heads * key_dim]")
+    rank = low_up.shape[0]
+    _f32_vector(low_bias, heads * key_dim, "gated_linear_attention: the decays' bias")
+    _need(0 <= low_off and low_off + rank <= proj.shape[1], "gated_linear_attention: the low-rank sums lie outside the rows")
+    return _linear_attention(LA_CHANNEL, proj, q_off, k_off, v_off, state, q_start, slots, heads, key_dim, value_dim, longest,
+                             dict(low_off=int(low_off), rank=rank, low_up=low_up.data_ptr(), low_bias=low_bias.data_ptr(), tau=float(tau),
+                                  q_scale=float(q_scale)))
+
+
+def matrix_memory(proj: torch.Tensor, q_off: int, k_off: int, v_off: int, i_off: int, f_off: int, i_bias: torch.Tensor,
+                  f_bias: torch.Tensor, cap: float, q_scale: float, state: torch.Tensor, q_start: torch.Tensor, slots: torch.Tensor,
+                  positions: torch.Tensor, heads: int, key_dim: int, value_dim: int, longest: int | None = None
+                  ) -> tuple[torch.Tensor, torch.Tensor]:
+    """The matrix memory of xLSTM (mLSTM) from the 32-bit sums ``proj``: q (times ``q_scale``), k and v as they are; per head
+    and token the log gates ``i = cap tanh((. + i_bias) / cap)`` and ``f = log sigmoid(cap tanh((. + f_bias) / cap))`` (sums
+    from ``i_off`` and ``f_off`` on); with the running maximum ``m' = max(f + m, i)``, ``S <- exp(f + m - m') S + exp(i - m')
+    k v^T`` and n likewise with k alone.  Returns what ``group_norm_gate`` takes as ``o`` and ``floor``: [tokens, heads * w]
+    with ``S^T q`` of a head and, behind it, ``n . q`` (w: value_dim + 1 rounded up to a multiple of 4), and exp(-m') [tokens, heads]."""
+    _gpu(i_bias, f_bias, positions)
+    _i32(positions, "positions")
+    _need(positions.numel() == proj.shape[0], "matrix_memory: one position a token")
+    _f32_vector(i_bias, heads, "matrix_memory: the input gate's bias")
+    _f32_vector(f_bias, heads, "matrix_memory: the forget gate's bias")
+    for off in (i_off, f_off):
+        _need(0 <= off and off + heads <= proj.shape[1], "matrix_memory: a gate's sums lie outside the rows")
+    floor = torch.empty((proj.shape[0], heads), dtype=torch.float32, device=proj.device)
+    o = _linear_attention(LA_MEMORY, proj, q_off, k_off, v_off, state, q_start, slots, heads, key_dim, value_dim, longest,
+                          dict(i_off=int(i_off), f_off=int(f_off), i_bias=i_bias.data_ptr(), f_bias=f_bias.data_ptr(), cap=float(cap),
+                               q_scale=float(q_scale), positions=positions.data_ptr(), floor=floor.data_ptr()),
+                          o_head=-(-(value_dim + 1) // 4) * 4)
+    return o, floor
 
 
 def group_norm_gate(o: torch.Tensor, weight: torch.Tensor, eps: float, groups: int, out_dtype: torch.dtype,
-                    gate: torch.Tensor | None = None, scale: float = 1.0, out: torch.Tensor | None = None) -> torch.Tensor:
+                    gate: torch.Tensor | None = None, scale: float = 1.0, out: torch.Tensor | None = None, size: int | None = None,
+                    floor: torch.Tensor | None = None, silu_gate: bool = False) -> torch.Tensor:
     """Every group's numbers of a token (``groups`` equal groups a row of the 32-bit ``o``) divided by their root
-    mean square, times ``weight`` (32-bit, one group's size, shared by the groups), times sigmoid(``gate``) where
-    one is given (32-bit, ``o``'s shape, rows a stride apart), times ``scale``; rounded once to ``out_dtype``.
-    ``out``: a 2-d view of that type to write to (rows a stride apart)."""
-    _gpu(o, weight, gate, out)
+    mean square, times ``weight`` (32-bit, one group's size, shared by the groups, or a whole row's), times sigmoid(``gate``)
+    (``silu_gate``: silu(``gate``)) where one is given (32-bit, the result's shape, rows a stride apart), times ``scale``;
+    rounded once to ``out_dtype``.  ``out``: a 2-d view of that type to write to (rows a stride apart).  ``size``: the
+    numbers of a group that count, the leading ones (by default all).  ``floor`` (32-bit [tokens, groups]): a group's numbers
+    are first divided by max(|d|, floor) + 1e-6 with d the number behind those that count."""
+    _gpu(o, weight, gate, out, floor)
+    groups = int(groups)
     _need(o.dim() == 2 and o.dtype == torch.float32 and o.is_contiguous() and o.shape[1] % groups == 0,
           "group_norm_gate: contiguous float32 rows of equal groups")
-    n, width = o.shape
-    size = width // int(groups)
-    _f32_vector(weight, size, "group_norm_gate: the weight")
-    _need(gate is None or (gate.shape == o.shape and gate.dtype == torch.float32 and gate.stride(1) == 1),
-          "group_norm_gate: a 32-bit gate of the rows' shape")
+    n, o_group = o.shape[0], o.shape[1] // groups
+    size = o_group if size is None else int(size)
+    width = groups * size
+    _need(0 < size <= o_group - (0 if floor is None else 1), "group_norm_gate: a group holds fewer numbers than that")
+    _need(weight.shape in ((size,), (width,)), f"group_norm_gate: a weight of {size} or {width} numbers")
+    _f32_vector(weight, weight.numel(), "group_norm_gate: the weight")
+    _need(floor is None or (floor.shape == (n, groups) and floor.dtype == torch.float32 and floor.is_contiguous()),
+          "group_norm_gate: the floors must be contiguous float32 [tokens, groups]")
+    _need(gate is None or (gate.shape == (n, width) and gate.dtype == torch.float32 and gate.stride(1) == 1),
+          "group_norm_gate: a 32-bit gate of the result's shape")
     if out is None:
         out = torch.empty((n, width), dtype=out_dtype, device=o.device)
     _need(out.shape == (n, width) and out.dtype == out_dtype and out.stride(1) == 1, "group_norm_gate: the result's view")
     if n:
-        call("tk_group_norm_gate", dtype_code(out_dtype), o.data_ptr(), gate.data_ptr() if gate is not None else None,
-             gate.stride(0) if gate is not None else 0, weight.data_ptr(), float(eps), float(scale), out.data_ptr(), out.stride(0),
-             n, int(groups), size, _stream())
+        call("tk_group_norm_gate", dtype_code(out_dtype), o.data_ptr(), o_group, gate.data_ptr() if gate is not None else None,
+             gate.stride(0) if gate is not None else 0, 1 if silu_gate else 0, weight.data_ptr(), 1 if weight.numel() != size else 0,
+             floor.data_ptr() if floor is not None else None, float(eps), float(scale), out.data_ptr(), out.stride(0),
+             n, groups, size, _stream())
     return out
 
 
@@ -1724,7 +1815,7 @@ def attention_tile_f32(
     sink: torch.Tensor | None = None, split: bool | None = None, key_chunk: int = 0, longest: int = 0, first_row: int = 0,
     score_bias: torch.Tensor | None = None, value_freq: torch.Tensor | None = None,
     value_pair_halves: bool = False, gate: torch.Tensor | None = None, softcap: float = 0.0,
-    distance_bias: "DistanceBias | None" = None,
+    distance_bias: "DistanceBias | None" = None, section: int = 0,
 ) -> torch.Tensor:
     """Attention in 32-bit arithmetic on the matrix cores: every token of the step over its
     request's pages; ``tile_req`` / ``tile_row0`` name each tile's request and its first token's
@@ -1738,7 +1829,7 @@ def attention_tile_f32(
     ``first_row``: ``q`` holds the step's rows from this one on only (the tiles name none before it), and so
     does the result.  ``score_bias``: sigmoid weights as in ``paged_attention_generic``.  ``value_freq``,
     ``value_pair_halves``, ``gate``: what ``unrotate_gate_`` does, in the kernel's own epilogue (halves only where
-    ``attention_tile_turns_halves``)."""
+    ``attention_tile_turns_halves``).  ``section`` as in ``paged_attention_generic``."""
     _gpu(q, kcache, vcache, block_table, q_start, kv_len, tile_req, tile_row0, sink, score_bias, value_freq, gate)
     db = _checked_distance_bias(distance_bias, nq)
     _f32_vector(value_freq, value_dim // 2, "attention: the values' frequencies")
@@ -1767,11 +1858,13 @@ def attention_tile_f32(
         # (behind a window a tile sees at most window + 15 keys, whatever the request's length: they lie in
         # `seen // chunk + 1` chunks at most, one more when they start inside one, and the kernel counts a tile's
         # chunks from the first it sees)
-        seen = min(int(longest), int(window) + 15) if window > 0 else int(longest)
+        # (the same for a tile whose first token is the last of its section)
+        reach = int(section) or int(window)
+        seen = min(int(longest), reach + 15) if reach > 0 else int(longest)
         while key_chunk < ATTENTION_TILE_LONGEST_CHUNK and groups * -(-seen // (2 * key_chunk)) >= ATTENTION_TILE_WORKGROUPS:
             key_chunk *= 2
         chunks = -(-int(longest) // int(key_chunk))
-        if window > 0:
+        if reach > 0:
             chunks = min(chunks, -(-seen // int(key_chunk)) + 1)
         words = load("core").tk_attention_tile_part_words(value_dim)
         part = torch.empty((tile_req.numel() * nkv * ((nq // nkv) // int(heads_a_tile)) * chunks * words,), dtype=torch.float32, device=q.device)
@@ -1781,7 +1874,7 @@ def attention_tile_f32(
     call("tk_attention_tile_f32", dtype_code(q.dtype), q_base, q.stride(0), out_base, out.stride(0),
          kcache.data_ptr(), vcache.data_ptr(), block_table.data_ptr(), block_table.stride(0), q_start.data_ptr(),
          kv_len.data_ptr(), tile_req.data_ptr(), tile_row0.data_ptr(), tile_req.numel(), nq, nkv, key_dim, value_dim,
-         page_size, int(window), float(scale), sink.data_ptr() if sink is not None else None,
+         page_size, int(window), int(section), float(scale), sink.data_ptr() if sink is not None else None,
          score_bias.data_ptr() if score_bias is not None else None, int(heads_a_tile),
          1 if split else 0, int(key_chunk) if chunks else 0, chunks, part.data_ptr() if part is not None else None,
          value_freq.data_ptr() if value_freq is not None else None, 1 if value_pair_halves else 0,
@@ -1906,27 +1999,37 @@ def gated_head_norm(o: torch.Tensor, gate: torch.Tensor, weight: torch.Tensor, e
 
 def post_norm_residual(x: torch.Tensor, branch: torch.Tensor, branch_weight: torch.Tensor, branch_eps: float,
                        weight: torch.Tensor | None = None, eps: float = 0.0, out_dtype: torch.dtype = torch.float32,
-                       in_place: bool = True, plain_rows: bool = False) -> tuple[torch.Tensor, torch.Tensor | None]:
+                       in_place: bool = True, plain_rows: bool = False, second: "tuple[torch.Tensor, torch.Tensor] | None" = None,
+                       mult: float = 1.0) -> tuple[torch.Tensor, torch.Tensor | None]:
     """``x_new = x + branch / sqrt(mean(branch^2) + branch_eps) * branch_weight`` on a 32-bit
     stream (the branch 32-bit too), and, when ``weight`` is given, the rows of the norm that
     reads the new stream, ``x_new / sqrt(mean(x_new^2) + eps) * weight`` rounded once to
     ``out_dtype``.  Returns (x_new, those rows or None).  ``in_place``: x_new overwrites x.
     ``plain_rows`` (without ``weight``): the rows returned are x_new itself rounded once to ``out_dtype``
-    (x_new when that is 32-bit): for sublayers that read the stream unnormed."""
-    _gpu(x, branch, branch_weight, weight)
-    _need(x.dim() == 2 and x.dtype == torch.float32 and x.is_contiguous(), "post_norm_residual: the stream must be contiguous float32 [rows, H]")
-    _need(branch.shape == x.shape and branch.dtype == torch.float32 and branch.is_contiguous(),
+    (x_new when that is 32-bit): for sublayers that read the stream unnormed.  ``second``: (rows, weight) of a branch
+    beside the first; ``x_new = x + mult * (both, each normed)``, and ``x`` may be None for zeros."""
+    _gpu(x, branch, branch_weight, weight, *(second or ()))
+    _need(x is not None or (second is not None and not in_place), "post_norm_residual: only two branches may stand alone, in new rows")
+    _need(x is None or (x.dim() == 2 and x.dtype == torch.float32 and x.is_contiguous()), "post_norm_residual: the stream must be contiguous float32 [rows, H]")
+    _need(second is not None or float(mult) == 1.0, "post_norm_residual: a factor goes with a second branch")
+    for y in ([branch, second[0]] if second is not None and x is None else [second[0]] if second is not None else []):
+        _need(y.shape == branch.shape and y.dim() == 2 and y.dtype == torch.float32 and y.is_contiguous(),
+              "post_norm_residual: the branches must be contiguous float32 of one shape")
+    _need(x is None or branch.shape == x.shape and branch.dtype == torch.float32 and branch.is_contiguous(),
           "post_norm_residual: the branch must be contiguous float32 of the stream's shape")
-    rows, hidden = x.shape
+    rows, hidden = branch.shape
     _f32_vector(branch_weight, hidden, "post_norm_residual: the branch norm's weight")
+    if second is not None:
+        _f32_vector(second[1], hidden, "post_norm_residual: the second branch norm's weight")
     _f32_vector(weight, hidden, "post_norm_residual: a norm weight")
-    x_out = x if in_place else torch.empty_like(x)
+    x_out = x if in_place else torch.empty_like(branch)
     _need(not (plain_rows and weight is not None), "post_norm_residual: plain rows or a norm's rows, not both")
     cast = plain_rows and out_dtype != torch.float32
-    h = torch.empty((rows, hidden), dtype=out_dtype, device=x.device) if (weight is not None or cast) else None
+    h = torch.empty((rows, hidden), dtype=out_dtype, device=branch.device) if (weight is not None or cast) else None
     if rows:
-        call("tk_post_norm_residual", dtype_code(out_dtype), x.data_ptr(), branch.data_ptr(), branch_weight.data_ptr(),
-             float(branch_eps), x_out.data_ptr(), weight.data_ptr() if weight is not None else None, float(eps),
+        call("tk_post_norm_residual", dtype_code(out_dtype), x.data_ptr() if x is not None else None, branch.data_ptr(),
+             branch_weight.data_ptr(), float(branch_eps), second[0].data_ptr() if second is not None else None,
+             second[1].data_ptr() if second is not None else None, float(mult), x_out.data_ptr(), weight.data_ptr() if weight is not None else None, float(eps),
              h.data_ptr() if h is not None else None, rows, hidden, _stream())
     return x_out, (x_out if plain_rows and not cast else h)
 
@@ -1991,7 +2094,8 @@ def head_linear(x: torch.Tensor, w: torch.Tensor, out_f32: bool = False, positio
         # many rows: tiles of 32 rows on the matrix cores, the head as the tile's group
         tiles = -(-x.shape[0] // GROUPED_TILE)
         call("tk_grouped_gemm_bf16", x.data_ptr(), x.stride(0), None, None, None, tiles, heads, n_in, n_out, w.data_ptr(),
-             n_out * n_in, y.data_ptr(), y.stride(0), n_out, n_in, x.shape[0], 0, 1 if out_f32 else 0, None, None, GROUPED_TILE, _stream())
+             n_out * n_in, y.data_ptr(), y.stride(0), n_out, n_in, x.shape[0], 0, 1 if out_f32 else 0, None, None, GROUPED_TILE, 0.0, 0.0,
+             _stream())
         return y
     if freq is not None:
         _i32(positions, "positions")
@@ -2038,14 +2142,52 @@ def expert_route(h: torch.Tensor, w_router: torch.Tensor, correction: torch.Tens
     return ids, weights, gate
 
 
-def expert_mix(h: torch.Tensor, w_gate_up: torch.Tensor, w_down: torch.Tensor, ids: torch.Tensor, weights: torch.Tensor,
+class ExpertTables:
+    """Tables of experts by token id, one a layer (int32 [vocab, top]), as ``expert_lookup`` reads them."""
+
+    def __init__(self, tables: "list[torch.Tensor]"):
+        _gpu(*tables)
+        self.tables = list(tables)
+        self.vocab = tables[0].shape[0]
+        words, at = [], 0
+        self.spans: list[tuple[int, int]] = []  # per layer: its top and where its part begins, in numbers a token
+        for t in tables:
+            _i32(t, "a table of experts")
+            _need(t.dim() == 2 and t.shape[0] == self.vocab, "tables of experts: one row a token id")
+            top = t.shape[1]
+            words.append([t.data_ptr(), top | (at << 32)])
+            self.spans.append((top, at))
+            at += top
+        self.total = at
+        self.layers = torch.tensor(words, dtype=torch.int64).to(tables[0].device)
+
+
+def expert_lookup(token_ids: torch.Tensor, last_token: torch.Tensor | None, tables: ExpertTables) -> "list[torch.Tensor]":
+    """The chosen experts of every token of a step for every layer's table, [tokens, top] int32 each, in one launch; a token id
+    below 0 is read from ``last_token`` [-id - 1]."""
+    _gpu(token_ids, last_token, tables.layers)
+    _i32(token_ids, "token ids")
+    if last_token is not None:
+        _i32(last_token, "last_token")
+    n = token_ids.numel()
+    ids = torch.empty((n * tables.total,), dtype=torch.int32, device=token_ids.device)
+    call("tk_expert_lookup", token_ids.data_ptr(), last_token.data_ptr() if last_token is not None else None, tables.vocab,
+         tables.layers.data_ptr(), ids.data_ptr(), len(tables.tables), n, _stream())
+    return [ids[at * n : (at + top) * n].view(n, top) for top, at in tables.spans]
+
+
+def expert_mix(h: torch.Tensor, w_gate_up: torch.Tensor, w_down: torch.Tensor, ids: torch.Tensor, weights: torch.Tensor | None,
                shared: torch.Tensor | None = None, shared_gate: torch.Tensor | None = None,
-               weights_on_input: bool = False) -> torch.Tensor:
+               weights_on_input: bool = False, glu: "tuple[float, float] | None" = None) -> torch.Tensor:
     """The weighted sum of a token's chosen experts, 32-bit [tokens, width]: expert e is
     ``w_down[e] (silu(gate) * up)`` with [gate | up] = ``w_gate_up[e] h``; an id from
     ``len(w_down)`` on names an identity expert (its output is h), a negative id an empty
     place.  ``shared`` (32-bit [tokens, width]) times ``shared_gate`` [tokens] is added.  ``weights_on_input``: a chosen
-    expert reads weight * h and its output is added as it is (the factor goes on the 32-bit sums of gate and up)."""
+    expert reads weight * h and its output is added as it is (the factor goes on the 32-bit sums of gate and up).  ``glu``:
+    (limit, alpha) of the gated activation with clamps, in place of silu(gate) * up.  ``weights`` None: equal parts."""
+    _need(weights is not None or not weights_on_input, "expert_mix: equal parts multiply the experts' outputs")
+    limit, alpha = (0.0, 0.0) if glu is None else (float(glu[0]), float(glu[1]))
+    _need(glu is None or limit > 0.0, "expert_mix: the clamps' limit must be positive")
     unit = 1 if weights_on_input else 0
     on_input = weights.data_ptr() if weights_on_input else None
     _gpu(h, w_gate_up, w_down, ids, weights, shared, shared_gate)
@@ -2057,12 +2199,13 @@ def expert_mix(h: torch.Tensor, w_gate_up: torch.Tensor, w_down: torch.Tensor, i
     n = h.shape[0]
     _i32(ids, "ids")
     top = ids.shape[1]
-    _need(ids.shape == (n, top) and weights.shape == (n, top) and weights.dtype == torch.float32 and weights.is_contiguous(),
+    _need(ids.shape == (n, top) and (weights is None or weights.shape == (n, top) and weights.dtype == torch.float32 and weights.is_contiguous()),
           "expert_mix: ids and weights [tokens, top]")
     if shared is not None:
         _need(shared.shape == (n, width) and shared.dtype == torch.float32 and shared.is_contiguous(), "expert_mix: the shared expert's rows must be float32 [tokens, width]")
         _f32_vector(shared_gate, n, "expert_mix: the shared expert's gate")
     out = torch.empty((n, width), dtype=torch.float32, device=h.device)
+    weight_ptr = weights.data_ptr() if weights is not None else None
     if n == 0:
         return out
     if n > GROUPED_FROM_ROWS and _grouped_takes(h, w_gate_up, width) and ff % 8 == 0 and w_down.data_ptr() % 16 == 0:
@@ -2077,18 +2220,18 @@ def expert_mix(h: torch.Tensor, w_gate_up: torch.Tensor, w_down: torch.Tensor, i
         inter = torch.empty((slots, ff), dtype=h.dtype, device=h.device)
         call("tk_grouped_gemm_bf16", h.data_ptr(), h.stride(0), slot_token.data_ptr(), None, tile_group.data_ptr(), max_tiles, 0,
              0, 0, w_gate_up.data_ptr(), 2 * ff * width, inter.data_ptr(), ff, ff, width, slots, 1, 0, on_input,
-             slot_pair.data_ptr() if weights_on_input else None, tile, _stream())
+             slot_pair.data_ptr() if weights_on_input else None, tile, limit, alpha, _stream())
         y = torch.empty((n * top, width), dtype=h.dtype, device=h.device)
         call("tk_grouped_gemm_bf16", inter.data_ptr(), ff, None, slot_pair.data_ptr(), tile_group.data_ptr(), max_tiles, 0,
-             0, 0, w_down.data_ptr(), width * ff, y.data_ptr(), width, width, ff, slots, 0, 0, None, None, tile, _stream())
-        call("tk_expert_sum", h.data_ptr(), h.stride(0), y.data_ptr(), ids.data_ptr(), weights.data_ptr(),
+             0, 0, w_down.data_ptr(), width * ff, y.data_ptr(), width, width, ff, slots, 0, 0, None, None, tile, 0.0, 0.0, _stream())
+        call("tk_expert_sum", h.data_ptr(), h.stride(0), y.data_ptr(), ids.data_ptr(), weight_ptr,
              shared.data_ptr() if shared is not None else None, shared_gate.data_ptr() if shared is not None else None,
              out.data_ptr(), n, width, experts, top, unit, _stream())
         return out
     inter = torch.empty((n * top, ff), dtype=h.dtype, device=h.device)
     call("tk_expert_gate_up", dtype_code(h.dtype), h.data_ptr(), h.stride(0), w_gate_up.data_ptr(), ids.data_ptr(), on_input,
-         inter.data_ptr(), n, width, ff, experts, top, _stream())
+         inter.data_ptr(), n, width, ff, experts, top, limit, alpha, _stream())
     call("tk_expert_combine", dtype_code(h.dtype), h.data_ptr(), h.stride(0), inter.data_ptr(), w_down.data_ptr(),
-         ids.data_ptr(), weights.data_ptr(), shared.data_ptr() if shared is not None else None,
+         ids.data_ptr(), weight_ptr, shared.data_ptr() if shared is not None else None,
          shared_gate.data_ptr() if shared is not None else None, out.data_ptr(), n, width, ff, experts, top, unit, _stream())
     return out

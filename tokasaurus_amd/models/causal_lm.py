@@ -83,12 +83,16 @@ class CausalLM:
         """Run the batch of ``ctx`` and return logits [len(want_rows), vocab] in 32-bit;
         ``want_rows`` None stands for every row in order (no rows are picked out then).
         ``logits_out``: a contiguous buffer of that shape that receives the logits and is returned."""
+        # (what parts share over the layers and compute once a step)
+        for start in self.shared.get("step_starts", ()):
+            start(ctx)
         # (an embedding may already have made the rows of the first block's entry norm)
         x, prepared = stream_and_prepared(self.embedding.forward(ctx))
         order = self.spec.run_order
         last = len(order) - 1
         # a connector reads the embedding's output again; blocks may update the stream in place
-        x0 = (x.clone() if any(not getattr(c, "takes_history", False) and not c.updates_stream for c in self.connectors) else None)
+        x0 = (x.clone() if any(not getattr(c, "takes_history", False) and (c.reads_embedding or not c.updates_stream)
+                               for c in self.connectors) else None)
         # connectors that read every stream so far: the embedding's output and each block's result are kept side by
         # side, [streams, tokens, H]; a block updates its input in place, so its input is a copy in the next place
         hist = None
@@ -105,7 +109,9 @@ class CausalLM:
             rows = want_rows if i == last else None
             block = self.blocks[entry.layer]
             if entry.before is not None and self.connectors[entry.before].updates_stream:
-                out = self.connectors[entry.before].update(x, handed, block.entry_norm() if block.fuses_norm else None)
+                before = self.connectors[entry.before]
+                more = {"x0": x0} if before.reads_embedding else {}
+                out = before.update(x, handed, block.entry_norm() if block.fuses_norm else None, **more)
                 (x, prepared), handed = stream_and_prepared(out), None
             elif entry.before is not None:
                 x, prepared = self.connectors[entry.before].forward(x, x0), None

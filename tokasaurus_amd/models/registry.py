@@ -22,6 +22,8 @@ from tokasaurus_amd.config.sazilorn_config import SazilornConfig
 from tokasaurus_amd.models.sazilorn import sazilorn_spec
 from tokasaurus_amd.config.vekasun_config import VekasunConfig
 from tokasaurus_amd.models.vekasun import vekasun_spec
+from tokasaurus_amd.config.tefavik_config import TefavikConfig
+from tokasaurus_amd.models.tefavik import tefavik_spec
 from tokasaurus_amd.models.spec import ModelSpec
 
 
@@ -50,6 +52,7 @@ register_architecture(Architecture("taborax", TaboraxConfig.from_dict, taborax_s
 register_architecture(Architecture("sakevik", SakevikConfig.from_dict, sakevik_spec, class_names=("Sakevik",)))
 register_architecture(Architecture("sazilorn", SazilornConfig.from_dict, sazilorn_spec, class_names=("Sazilorn",)))
 register_architecture(Architecture("vekasun", VekasunConfig.from_dict, vekasun_spec, class_names=("Vekasun",)))
+register_architecture(Architecture("tefavik", TefavikConfig.from_dict, tefavik_spec, class_names=("Tefavik",)))
 
 
 def architecture_of(config_dict: dict[str, Any]) -> Architecture:

@@ -40,6 +40,7 @@ class TensorSpec:
     name: str
     shape: tuple[int, ...]
     kind: str = MATRIX
+    below: int = 0  # integer tables: every row holds different numbers from 0 to below - 1 (0: any numbers)
 
 
 @dataclass(frozen=True)
@@ -51,10 +52,26 @@ class CacheNeed:
     head_dim: int
     window: int = 0  # 0: every key is kept; > 0: only the last `window` positions are read
     value_dim: int = 0  # size of a value head where it differs from a key head's (0: the same)
+    section: int = 0  # > 0 (without a window): a query reads only keys of its own section of this many positions
+
+    def __post_init__(self):
+        if self.window and self.section:
+            raise ValueError("keys are read within a window or within sections, not both")
 
     @property
     def value_size(self) -> int:
         return self.value_dim or self.head_dim
+
+    @property
+    def keeps_all(self) -> bool:
+        """Whether a request's keys stay until it ends (else pages go back while it runs)."""
+        return not self.window and not self.section
+
+    def first_read(self, new_len: int) -> int:
+        """The first position that a query at position ``new_len`` or later can read."""
+        if self.section:
+            return new_len // self.section * self.section
+        return max(0, new_len - self.window + 1) if self.window else 0
 
 
 @dataclass(frozen=True)
@@ -164,6 +181,24 @@ class Normed:
         return self.norm.forward(self.x)
 
 
+@dataclass
+class NormedSum:
+    """``mult * (rms_norm(a) * wa + rms_norm(b) * wb)`` of two 32-bit branches, not computed yet: whoever adds it to a stream
+    norms, sums and adds in one pass.  ``rows()`` computes it alone."""
+
+    a: torch.Tensor
+    wa: torch.Tensor
+    b: torch.Tensor
+    wb: torch.Tensor
+    eps: float
+    mult: float
+
+    def rows(self) -> torch.Tensor:
+        from tokasaurus_amd.kernels import ops
+
+        return ops.post_norm_residual(None, self.a, self.wa, self.eps, in_place=False, second=(self.b, self.wb), mult=self.mult)[0]
+
+
 # --------------------------------------------------------------------------
 # interfaces
 # --------------------------------------------------------------------------
@@ -210,9 +245,13 @@ class Mixer(Part):
     A mixer (or feed-forward) with ``fuses_norm = True`` takes ``h`` as a ``Normed``
     and a keyword ``emit_norm`` (the norm that will be applied to its result, or
     None) and may return ``(stream, Prepared)`` instead of the stream alone.
+
+    A mixer with ``gives_normed_sum = True`` also has ``normed_sum(h, ctx, cache, state, rows)``, which returns
+    what ``mix`` returns as a ``NormedSum``: for a block that can add it to the stream in one pass.
     """
 
     fuses_norm = False
+    gives_normed_sum = False
 
     def cache_need(self) -> CacheNeed | None:
         return None
@@ -251,9 +290,13 @@ class Mixer(Part):
 
 
 class FeedForward(Part):
-    """Token-wise transformation: returns ``residual + ff(h)`` (see ``Mixer`` for ``fuses_norm``)."""
+    """Token-wise transformation: returns ``residual + ff(h)`` (see ``Mixer`` for ``fuses_norm``).
+    One that reads the tokens' ids beside their rows says ``reads_tokens = True`` and takes two more keywords,
+    ``ctx`` (the step) and ``rows`` (the step's rows that ``h`` holds, None: all of them); blocks that hand
+    them over say so."""
 
     fuses_norm = False
+    reads_tokens = False
 
     def forward(self, h: torch.Tensor, residual: torch.Tensor) -> torch.Tensor:
         raise NotImplementedError
@@ -297,9 +340,11 @@ class Connector(Part):
     runs before it (``models.spec.RunEntry.before``).  A connector that reads the stream alone says
     ``updates_stream = True`` and has ``update(x, pending, next_norm)`` instead: it changes ``x`` in place, adds
     the branch that the block in front has handed over unsummed (``parts.block.PendingSum`` or None) in the same pass,
-    and may return (stream, ``Prepared``) for the norm that reads it."""
+    and may return (stream, ``Prepared``) for the norm that reads it.  One that does so and reads the embedding's output too
+    says ``reads_embedding = True`` and gets it as the keyword ``x0``."""
 
     updates_stream = False
+    reads_embedding = False
 
     def forward(self, x: torch.Tensor, x0: torch.Tensor) -> torch.Tensor:
         raise NotImplementedError

@@ -23,6 +23,7 @@ from tokasaurus_amd.parts.base import (
     CacheView,
     Connector,
     Normed,
+    NormedSum,
     Part,
     Prepared,
     PartSpec,
@@ -45,6 +46,13 @@ def build_with_shared(registry, spec: PartSpec, shared: dict):
 def stream_and_prepared(out) -> tuple[torch.Tensor, Prepared | None]:
     """A part returns the stream alone, or the stream with what it prepared for the next norm."""
     return out if isinstance(out, tuple) else (out, None)
+
+
+def transformed(feed_forward, h: torch.Tensor, ctx: StepContext, rows: torch.Tensor | None) -> torch.Tensor:
+    """The feed-forward's 32-bit output for the step's rows ``rows`` (None: all), handing over the step where it reads the tokens."""
+    if feed_forward.reads_tokens:
+        return feed_forward.transform(h, out_f32=True, ctx=ctx, rows=rows)
+    return feed_forward.transform(h, out_f32=True)
 
 
 @BLOCKS.register("pre_norm")
@@ -207,7 +215,7 @@ class ParallelResidualBlock(Block):
         if rows is not None:
             x = ops.gather_rows(x, rows)
             h2 = ops.gather_rows(h2, rows) if h2 is not None else None
-        b = self.feed_forward.transform(h2, out_f32=True) if self.feed_forward is not None else None
+        b = transformed(self.feed_forward, h2, ctx, rows) if self.feed_forward is not None else None
         if defer_sum:
             return PendingSum(x, (a, b), self.residual_mult)
         # the norms that read the new stream: the next block's pair or a single norm (the head's)
@@ -291,7 +299,7 @@ class SandwichNormBlock(Block):
         reader = self.ff_norm if self.feed_forward is not None else next_norm
         x, h = self._add(x, a, self.mixer_post_norm, reader)
         if self.feed_forward is not None:
-            b = self.feed_forward.transform(h, out_f32=True)
+            b = transformed(self.feed_forward, h, ctx, rows)
             reader = next_norm
             x, h = self._add(x, b, self.ff_post_norm, reader)
         if tap is not None:  # a list that collects the stream after every block (tests, debugging)
@@ -362,7 +370,7 @@ class PostNormBlock(Block):
         reader = self.entry if self.feed_forward is not None else next_norm
         x, h = self._add(x, a, self.mixer_post_norm, reader)
         if self.feed_forward is not None:
-            b = self.feed_forward.transform(h, out_f32=True)
+            b = transformed(self.feed_forward, h, ctx, rows)
             reader = next_norm
             x, h = self._add(x, b, self.ff_post_norm, reader)
         if tap is not None:  # a list that collects the stream after every block (tests, debugging)
@@ -374,7 +382,17 @@ class PostNormBlock(Block):
 
 def _update_stream(x: torch.Tensor, branches: tuple, reader, mult: float = 1.0, add_row: torch.Tensor | None = None):
     """x <- x + mult * (branches) + add_row on a 32-bit stream, in place, with the rows of the norm that reads it where
-    that norm can be written in the same pass (it has ``update``): (stream, ``Prepared`` or None)."""
+    that norm can be written in the same pass (it has ``update``): (stream, ``Prepared`` or None).  The first branch may be
+    a ``NormedSum``, alone: it is normed and added in the pass of a plain-weight RMS norm."""
+    if isinstance(branches[0], NormedSum):
+        s = branches[0]
+        assert branches[1] is None and mult == 1.0 and add_row is None, "a normed sum is added alone"
+        plain = getattr(reader, "same_rule", None) is not None and not reader.unit_offset
+        x, h = ops.post_norm_residual(x, s.a, s.wa, s.eps, reader.weight if plain else None, reader.eps if plain else 0.0,
+                                      reader.out_dtype if plain else torch.float32, second=(s.b, s.wb), mult=s.mult)
+        if plain:
+            return x, Prepared(None, reader, h)
+        branches = (None, None)
     if hasattr(reader, "update"):
         x, h = reader.update(x, branches, mult, add_row)
         return x, Prepared(None, reader, h)
@@ -388,7 +406,8 @@ class StreamPreNormBlock(Block):
     ``feed_forward`` (with its norm) may be absent.  The branches hand over their last products' 32-bit sums; one
     kernel adds a branch and writes the rows of the norm that reads the new stream (this block's second, the next
     block's first, or the head's).  The norms are any that have ``update`` (``stream_rmsnorm``, ``stream_layernorm``);
-    the mixer must have ``mix`` and the feed-forward ``transform``."""
+    the mixer must have ``mix`` (or ``normed_sum``) and the feed-forward ``transform``; a feed-forward that reads the
+    tokens' ids gets the step."""
 
     fuses_norm = True
     can_defer_sum = True
@@ -428,13 +447,18 @@ class StreamPreNormBlock(Block):
             h = prepared.normed
         else:
             h = self.mixer_norm.forward(x)
-        branch = self.mixer.mix(h, ctx, cache, state, rows, out_f32=True)
+        if self.mixer.gives_normed_sum:
+            branch = self.mixer.normed_sum(h, ctx, cache, state, rows)
+        else:
+            branch = self.mixer.mix(h, ctx, cache, state, rows, out_f32=True)
         if rows is not None:
             x = ops.gather_rows(x, rows)
         if self.feed_forward is not None:
             x, made = _update_stream(x, (branch, None), self.ff_norm)
-            branch = self.feed_forward.transform(made.normed, out_f32=True)
+            branch = transformed(self.feed_forward, made.normed, ctx, rows)
         if defer_sum:
+            if isinstance(branch, NormedSum):
+                branch = branch.rows()
             return PendingSum(x, (branch, None), 1.0)
         return _update_stream(x, (branch, None), next_norm)
 
@@ -465,6 +489,21 @@ class AddRow(Connector):
     def update(self, x: torch.Tensor, pending: "PendingSum | None", next_norm=None):
         branches, mult = (pending.branches, pending.mult) if pending is not None else ((None, None), 1.0)
         return _update_stream(x, branches, next_norm, mult, self.vector)
+
+
+@CONNECTORS.register("add_embedding")
+class AddEmbedding(Connector):
+    """x <- x + x0 on a 32-bit stream, x0 the embedding's output: in the pass that adds the branch of the block in front,
+    where that was handed over unsummed, and that writes the rows of the norm that reads the new stream."""
+
+    updates_stream = True
+    reads_embedding = True
+
+    def update(self, x: torch.Tensor, pending: "PendingSum | None", next_norm=None, x0: torch.Tensor | None = None):
+        a, b = pending.branches if pending is not None else (None, None)
+        if pending is not None and (b is not None or pending.mult != 1.0):
+            x, a = ops.residual_norm(x, (a, b), pending.mult)[0], None
+        return _update_stream(x, (a, x0), next_norm)
 
 
 @CONNECTORS.register("embedding_mix")

@@ -10,7 +10,8 @@ instead of neighbours, and values that are the keys themselves as projected, bef
 head with one weight for all heads; weights that are sigmoids of the biased scores instead of a
 softmax; values turned by their own position and the heads' results turned back by the query's; a
 sigmoid gate per head that reads the mixer's input; a soft cap on the scaled scores; a learned bias on the
-scores by (bucket of the distance, head); a sigmoid gate per element of the heads' results.
+scores by (bucket of the distance, head); a sigmoid gate per element of the heads' results; sections of positions
+that keep their keys to themselves.
 
 Scores, softmax weights, norms, angles and the rotation are 32-bit arithmetic in either storage
 type.  One kernel norms, rotates and appends (``ops.qk_prepare``); the attention itself runs on
@@ -88,6 +89,7 @@ class GroupedAttention(Mixer):
         softcap: float | None = None,
         distance_bias: dict | None = None,
         element_gate_name: str | None = None,
+        section: int = 0,
     ):
         """``names``: checkpoint names of the q, k, v, o matrices (k and v only with ``own_kv``).
         ``projection_norm``: ``{"q": name, "k": name, "eps": eps}``, weights of the whole
@@ -109,7 +111,12 @@ class GroupedAttention(Mixer):
         B, "far": D}``, a table [B, heads] of which row bucket(i - j) is added to the score of query i and key j (after
         the scale and the soft cap): distances below B / 2 have a bucket each, the others share the rest on a
         logarithmic scale that reaches the last bucket at D.  ``element_gate_name``: a matrix [heads * value_dim,
-        hidden]; the heads' results are multiplied element by element by sigmoid(gate h)."""
+        hidden]; the heads' results are multiplied element by element by sigmoid(gate h).  ``section``: positions are cut
+        at multiples of it, counted from a request's start, and a query sees only keys of its own section (0: all; not with
+        a window)."""
+        self.section = int(section)
+        if self.section and (window or cache_window):
+            raise ValueError("a window or sections, not both")
         self.softcap = float(softcap) if softcap else 0.0
         self.distance_bias = dict(distance_bias) if distance_bias else None
         self.element_gate_name = element_gate_name
@@ -198,7 +205,7 @@ class GroupedAttention(Mixer):
 
     def cache_need(self) -> CacheNeed:
         return CacheNeed(self.num_kv_heads, self.key_dim, self.cache_window,
-                         0 if self.value_dim == self.key_dim else self.value_dim)
+                         0 if self.value_dim == self.key_dim else self.value_dim, self.section)
 
     def check_cache(self, page_size: int, dtype: torch.dtype) -> None:
         ops.check_attention_shape(dtype, self.num_heads, self.num_kv_heads, self.key_dim, page_size,
@@ -268,13 +275,14 @@ class GroupedAttention(Mixer):
                                           window=self.window, scale=self.scale, sink=self.sink, key_chunk=self.key_chunk,
                                           longest=ctx.extras.get("kv_bound", ctx.max_kv_len), score_bias=self.score_bias,
                                           value_freq=self.value_freq if fused else None, value_pair_halves=v_halves,
-                                          gate=gate if fused else None, softcap=self.softcap, distance_bias=self.rel)
+                                          gate=gate if fused else None, softcap=self.softcap, distance_bias=self.rel,
+                                          section=self.section)
             after = after and not fused
         else:  # sizes that the matrix-core kernel does not take
             attn = ops.paged_attention_generic(qkv, cache.keys, cache.values, cache.block_table, ctx.token_req, ctx.positions,
                                                nq, nkv, dk, cache.page_size, window=self.window, scale=self.scale,
                                                value_dim=dv, sink=self.sink, score_bias=self.score_bias, softcap=self.softcap,
-                                               distance_bias=self.rel)
+                                               distance_bias=self.rel, section=self.section)
         if after:
             # the heads' results turned back by their own positions, then each head's gate
             ops.unrotate_gate_(attn, ctx.positions, self.value_freq, v_halves, gate, nq, dv)

@@ -11,6 +11,10 @@ the last ``identity`` router outputs have no tensors, their output is ``h`` itse
 expert of the same form may run for every token; its output is multiplied by
 ``sigmoid(w_sg . h)``, one number a token, where the checkpoint has such a gate, and added.
 
+Or there is no router at all (``table_experts``): a table of integers gives each token id its experts, in equal parts.  The
+choice then rests on the step's token ids alone and is looked up once a step for all layers.  An expert's activation may be the
+form with clamps, ``g sigmoid(alpha g) (u + 1)`` of ``g = min(gate, limit)`` and ``u = clamp(up, -limit, limit)``.
+
 One kernel routes (and computes the shared expert's gate); the experts' products run pair by
 pair (token, chosen expert), each a function of its own token only, and are summed per token
 in the order of the choice: a token's result does not depend on what else is in the batch.
@@ -21,12 +25,39 @@ from __future__ import annotations
 import torch
 
 from tokasaurus_amd.kernels import ops
-from tokasaurus_amd.parts.base import FEED_FORWARDS, MATRIX, SMALL_VECTOR, FeedForward, TensorSpec
+from tokasaurus_amd.parts.base import FEED_FORWARDS, INT_TABLE, MATRIX, SMALL_VECTOR, FeedForward, StepContext, TensorSpec
 from tokasaurus_amd.parts.linear import Linear, Placer
 
 
+class _Experts(FeedForward):
+    """The experts' matrices, one tensor for all experts of a layer."""
+
+    hidden_size: int
+    expert_size: int
+    num_experts: int
+    names: dict[str, str]
+    w_gate_up: torch.Tensor | None = None  # [experts, gate rows | up rows, hidden]
+    w_down: torch.Tensor | None = None  # [experts, hidden, expert_size]
+
+    def _expert(self, e: int, which: str) -> str:
+        return f"{self.names['expert'].format(e=e)}.{which}"
+
+    def _expert_specs(self) -> list[TensorSpec]:
+        W, F = self.hidden_size, self.expert_size
+        return [TensorSpec(self._expert(e, which), shape, MATRIX) for e in range(self.num_experts)
+                for which, shape in (("gate", (F, W)), ("up", (F, W)), ("down", (W, F)))]
+
+    def _load_experts(self, tensors: dict[str, torch.Tensor], placer: Placer) -> None:
+        n, E = self.names["expert"], range(self.num_experts)
+        self.w_gate_up = placer.place(("experts_gate_up", n), lambda: torch.stack(
+            [torch.cat([tensors[self._expert(e, "gate")], tensors[self._expert(e, "up")]], dim=0) for e in E]).to(
+                placer.dtype).contiguous().to(placer.device))
+        self.w_down = placer.place(("experts_down", n), lambda: torch.stack([tensors[self._expert(e, "down")] for e in E]).to(
+            placer.dtype).contiguous().to(placer.device))
+
+
 @FEED_FORWARDS.register("routed_experts")
-class RoutedExperts(FeedForward):
+class RoutedExperts(_Experts):
     def __init__(self, hidden_size: int, expert_size: int, num_experts: int, top: int, names: dict[str, str],
                  identity: int = 0, groups: int = 1, keep: int = 1, shared_size: int | None = None,
                  normalize_scale: float | None = None, scores: str = "softmax", weights_on_input: bool = False):
@@ -54,19 +85,14 @@ class RoutedExperts(FeedForward):
             sp = names["shared"]
             self.shared_gate_up = Linear(hidden_size, [f"{sp}.gate", f"{sp}.up"], [self.shared_size] * 2)
             self.shared_down = Linear(self.shared_size, [f"{sp}.down"], [hidden_size])
-        self.router = self.correction = self.w_gate_up = self.w_down = self.shared_gate = None
-
-    def _expert(self, e: int, which: str) -> str:
-        return f"{self.names['expert'].format(e=e)}.{which}"
+        self.router = self.correction = self.shared_gate = None
 
     def tensor_specs(self) -> list[TensorSpec]:
-        W, F = self.hidden_size, self.expert_size
+        W = self.hidden_size
         specs = [TensorSpec(self.names["router"], (self.n_all, W), MATRIX)]
         if self.names.get("correction"):
             specs.append(TensorSpec(self.names["correction"], (self.n_all,), SMALL_VECTOR))
-        for e in range(self.num_experts):
-            specs += [TensorSpec(self._expert(e, "gate"), (F, W), MATRIX), TensorSpec(self._expert(e, "up"), (F, W), MATRIX),
-                      TensorSpec(self._expert(e, "down"), (W, F), MATRIX)]
+        specs += self._expert_specs()
         if self.shared_size:
             specs += self.shared_gate_up.tensor_specs() + self.shared_down.tensor_specs()
             if self.names.get("shared_gate"):
@@ -74,7 +100,7 @@ class RoutedExperts(FeedForward):
         return specs
 
     def load(self, tensors: dict[str, torch.Tensor], placer: Placer) -> None:
-        n, E = self.names, self.num_experts
+        n = self.names
 
         def place(key, make):
             return placer.place(key, lambda: make().contiguous().to(placer.device))
@@ -82,11 +108,7 @@ class RoutedExperts(FeedForward):
         self.router = place(("row_major", n["router"]), lambda: tensors[n["router"]].to(placer.dtype))
         if n.get("correction"):
             self.correction = place(("vector_f32", n["correction"]), lambda: tensors[n["correction"]].to(torch.float32))
-        # one tensor for all experts: [experts, gate rows | up rows, hidden] and [experts, hidden, expert_size]
-        self.w_gate_up = place(("experts_gate_up", n["expert"]), lambda: torch.stack(
-            [torch.cat([tensors[self._expert(e, "gate")], tensors[self._expert(e, "up")]], dim=0) for e in range(E)]).to(placer.dtype))
-        self.w_down = place(("experts_down", n["expert"]), lambda: torch.stack(
-            [tensors[self._expert(e, "down")] for e in range(E)]).to(placer.dtype))
+        self._load_experts(tensors, placer)
         if self.shared_size:
             self.shared_gate_up.load(tensors, placer)
             self.shared_down.load(tensors, placer)
@@ -104,3 +126,64 @@ class RoutedExperts(FeedForward):
 
     def forward(self, h: torch.Tensor, residual: torch.Tensor):
         return ops.add(self.transform(h), residual.contiguous())
+
+
+class TokenTables:
+    """The tables of a model's layers whose experts go by token id: they are read once a step, for all layers, in front
+    of the embedding."""
+
+    KEY = "experts_by_token"  # in ``StepContext.extras``: per table the step's ids [tokens, top]
+
+    def __init__(self):
+        self.tables: list[torch.Tensor] = []
+        self._ready: "ops.ExpertTables | None" = None
+
+    def add(self, table: torch.Tensor) -> int:
+        self.tables.append(table)
+        self._ready = None
+        return len(self.tables) - 1
+
+    def __call__(self, ctx: StepContext) -> None:
+        if self._ready is None:
+            self._ready = ops.ExpertTables(self.tables)
+        ctx.extras[self.KEY] = ops.expert_lookup(ctx.token_ids, ctx.last_token, self._ready)
+
+
+@FEED_FORWARDS.register("table_experts")
+class TableExperts(_Experts):
+    reads_tokens = True
+
+    def __init__(self, hidden_size: int, vocab_size: int, expert_size: int, num_experts: int, top: int, names: dict[str, str],
+                 glu: tuple[float, float] | None = None, shared: dict | None = None):
+        """``names``: ``table`` (integers [vocab_size, top], the entries of a row differ) and ``expert`` as in
+        ``routed_experts``.  ``glu``: (limit, alpha) of the activation with clamps (None: silu)."""
+        self.hidden_size, self.vocab_size, self.expert_size = hidden_size, int(vocab_size), int(expert_size)
+        self.num_experts, self.top = int(num_experts), int(top)
+        if not 0 < self.top <= self.num_experts:
+            raise ValueError(f"{self.top} of {self.num_experts} experts")
+        self.names = dict(names)
+        self.glu = tuple(float(x) for x in glu) if glu else None
+        shared = shared if shared is not None else {}
+        if "token_tables" not in shared:
+            shared["token_tables"] = TokenTables()
+            shared.setdefault("step_starts", []).append(shared["token_tables"])
+        self.tables: TokenTables = shared["token_tables"]
+        self.index: int | None = None
+
+    def tensor_specs(self) -> list[TensorSpec]:
+        return [TensorSpec(self.names["table"], (self.vocab_size, self.top), INT_TABLE, below=self.num_experts), *self._expert_specs()]
+
+    def load(self, tensors: dict[str, torch.Tensor], placer: Placer) -> None:
+        self._load_experts(tensors, placer)
+        name = self.names["table"]
+        self.index = self.tables.add(placer.place(("int_table", name), lambda: tensors[name].to(torch.int32).contiguous().to(placer.device)))
+
+    def transform(self, h: torch.Tensor, out_f32: bool = False, ctx: StepContext | None = None, rows: torch.Tensor | None = None):
+        ids = ctx.extras[TokenTables.KEY][self.index]
+        if rows is not None:
+            ids = ids.index_select(0, rows)
+        y = ops.expert_mix(h, self.w_gate_up, self.w_down, ids, None, glu=self.glu)
+        return y if out_f32 else y.to(h.dtype)
+
+    def forward(self, h: torch.Tensor, residual: torch.Tensor, ctx: StepContext | None = None, rows: torch.Tensor | None = None):
+        return ops.add(self.transform(h, ctx=ctx, rows=rows), residual.contiguous())

@@ -123,6 +123,10 @@ def read_tensors(
                         wrong_type.append((name, f"integer table stored as {t.dtype}"))
                         continue
                     t = t.to(torch.int32)
+                    below = wanted[name].below
+                    if below and t.numel() and not (0 <= int(t.min()) and int(t.max()) < below):
+                        wrong_type.append((name, f"integer table with numbers outside 0 .. {below - 1}"))
+                        continue
                 elif not t.is_floating_point():
                     wrong_type.append((name, f"float tensor stored as {t.dtype}"))
                     continue

@@ -5,7 +5,8 @@ inputs, tokasaurus/manager/input_building.py:14-100).
 Every matrix is drawn from N(0, 0.02), every norm weight from 1 + N(0, 0.01) (from N(0, 0.01)
 when it is stored around zero, as is a vector that only nudges), other learned vectors from N(0, 0.5),
 in 32-bit on the host, in the sorted order of the tensor names, from one
-generator seeded with ``seed``; integer tables are drawn uniformly.  Tensors are
+generator seeded with ``seed``; integer tables are drawn uniformly (rows of different
+numbers where the table names rows' choices from a few).  Tensors are
 stored in bfloat16, so the 32-bit engine, the bfloat16 engine and any plain
 implementation read exactly the same values.  A tied head is not drawn.
 """
@@ -54,6 +55,11 @@ def draw_tensors(
         elif spec.kind == AVERAGE_WEIGHT:
             n = max(1, spec.shape[-1])
             t = (1.0 + 0.1 * torch.randn(spec.shape, generator=gen, dtype=torch.float32, device=device)) / n
+        elif spec.kind == INT_TABLE and spec.below:
+            # every row: the first columns of a random order of 0 .. below - 1
+            keys = torch.rand((*spec.shape[:-1], spec.below), generator=gen, dtype=torch.float32, device=device)
+            out[spec.name] = keys.argsort(dim=-1)[..., : spec.shape[-1]].to(torch.int32).contiguous()
+            continue
         elif spec.kind == INT_TABLE:
             out[spec.name] = torch.randint(0, 1 << 15, spec.shape, generator=gen, dtype=torch.int32, device=device)
             continue
