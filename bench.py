@@ -82,13 +82,13 @@ def parse() -> argparse.Namespace:
                    help="instead of the decode steps, a case that shapes of one length do not show (prints its own line): "
                         "chunked-prefill: one prompt of --context tokens in portions of --portion tokens; "
                         "mixed-decode: decode steps of --batch - 1 requests of --short tokens beside one of --context tokens")
-    p.add_argument("--design", default=None, choices=["kupuzen", "taborax", "sakevik", "sazilorn", "vekasun"],
+    p.add_argument("--design", default=None, choices=["kupuzen", "taborax", "sakevik", "sazilorn", "vekasun", "tefavik"],
                    help="instead of the decode steps: prefill and decode of this design at layer sizes of --design-sizes "
                         "beside the Llama shape of equal width, heads, feed-forward and layers (prints its own line)")
     p.add_argument("--design-sizes", default="1b,3b", help="which sizes of DESIGN_SIZES, comma separated")
-    p.add_argument("--design-beside", default=None, choices=["llama", "kupuzen", "taborax", "sakevik", "sazilorn"],
+    p.add_argument("--design-beside", default=None, choices=["llama", "kupuzen", "taborax", "sakevik", "sazilorn", "vekasun"],
                    help="the model the --design comparison stands beside (by default the Llama shape; for sazilorn the Kupuzen "
-                        "of equal size and for vekasun the Taborax, the closest existing designs)")
+                        "of equal size, for vekasun the Taborax and for tefavik the Sazilorn, the closest existing designs)")
     p.add_argument("--design-only", action="store_true", help="the --design comparison without its Llama half (for profiles)")
     p.add_argument("--design-layers", type=int, default=8, help="layers of both models in the --design comparison")
     p.add_argument("--design-context", type=int, default=4096, help="context at which the --design decode steps end")
@@ -453,9 +453,29 @@ def vekasun_like(size: dict, layers: int) -> dict:
             "loop": {"start": 1, "stop": 3, "times": 2}, "layers": [latent if i % 3 == 1 else mamba for i in range(distinct)]}
 
 
+# A Tefavik of the same width, vocabulary and number of layer runs: gated linear attention (half the Llama heads of twice the
+# size, decays through 16) and, two to every such layer, soft-capped attention (the Llama heads, chunks of 1,024 positions)
+# beside a matrix memory (a quarter of the Llama heads of twice the size); every feed-forward a mixture whose eight experts by
+# token id together have the Llama inner size (32 experts); two inner layers are passed twice, so `layers` layer runs use
+# `layers - 2` layers' weights.
+def tefavik_like(size: dict, layers: int) -> dict:
+    ll = size["llama"]
+    H, G = ll["num_attention_heads"], ll["num_key_value_heads"]
+    d = ll["hidden_size"] // H
+    mixture = {"kind": "moe", "expert": {"ff": ll["intermediate_size"] // 8, "limit": 7.0}, "router": {"experts": 32, "top": 8}}
+    gla = {"type": "gla", "mlp": mixture, "mixer": {"heads": H // 2, "dim": 2 * d, "vdim": 2 * d, "tau": 16.0, "rank": 16}}
+    pair = {"type": "parallel", "mlp": mixture, "mixer": {
+        "left": {"heads": H, "kv_heads": G, "dim": d, "vdim": d, "scale": d ** -0.5, "softcap": 50.0, "mask": {"size": size["window"]},
+                 "rot": {"base": ll["rope_theta"], "dims": d}},
+        "right": {"heads": H // 4, "dim": 2 * d, "vdim": 2 * d, "gate_cap": 15.0}}}
+    distinct = max(layers - 2, 3)
+    return {"architecture": "Tefavik", "vocab": ll["vocab_size"], "width": ll["hidden_size"], "norm": {"eps": 1e-6},
+            "loop": {"start": 1, "stop": 3, "times": 2}, "layers": [gla if i % 3 == 0 else pair for i in range(distinct)]}
+
+
 DESIGN_MODELS = {"kupuzen": kupuzen_like, "taborax": taborax_like, "sakevik": sakevik_like, "sazilorn": sazilorn_like,
-                 "vekasun": vekasun_like}
-DESIGN_BESIDE = {"sazilorn": "kupuzen", "vekasun": "taborax"}  # the closest existing design where that is not the Llama shape
+                 "vekasun": vekasun_like, "tefavik": tefavik_like}
+DESIGN_BESIDE = {"sazilorn": "kupuzen", "vekasun": "taborax", "tefavik": "sazilorn"}  # the closest existing design where that is not the Llama shape
 
 
 def run_design(args) -> int:
