@@ -45,7 +45,7 @@ def i32(v):
 # ---------------------------------------------------------------------------------- kernels alone
 
 
-def cuts_of(lens, longest_first):
+def cuts_of(lens):
     """The same requests' tokens as steps: whole; two portions; portions of a few tokens and single tokens."""
     yield [list(lens)]
     yield [[max(1, n // 2) for n in lens], [n - max(1, n // 2) for n in lens]]
@@ -59,8 +59,8 @@ def cuts_of(lens, longest_first):
         yield steps
 
 
-def walk(run, proj, lens, slots, steps):
-    """Hand ``run`` the rows of every step (rows, q_start, slots, positions, longest) and put its results back in the order of proj."""
+def walk(run, proj, lens, slots, steps, in_chunks):
+    """Hand ``run`` the rows of every step (rows, q_start, slots, positions, longest, chunks) and put its results back in the order of proj."""
     starts = [sum(lens[:r]) for r in range(len(lens))]
     held = [0] * len(lens)
     out = None
@@ -74,7 +74,13 @@ def walk(run, proj, lens, slots, steps):
             q_start.append(len(idx))
             used.append(slots[r])
             held[r] += n
-        got = run(proj[idx].contiguous().cuda(), i32(q_start), i32(used), i32(pos), max(sizes))
+        req, row0, first = [], [], [0]
+        for r, (a, b) in enumerate(zip(q_start, q_start[1:])):
+            req += [r] * len(range(a, b, 64))
+            row0 += range(a, b, 64)
+            first.append(len(req))
+        chunks = ops.ChunkPlan(i32(req), i32(row0), i32(first)) if in_chunks else None
+        got = run(proj[idx].contiguous().cuda(), i32(q_start), i32(used), i32(pos), max(sizes), chunks)
         got = [g.cpu() for g in got]
         if out is None:
             out = [torch.zeros(proj.shape[0], g.shape[1]) for g in got]
@@ -91,8 +97,10 @@ LINEAR_CASES = [  # heads, key size, value size, lengths of the requests
 
 @pytest.mark.parametrize("heads, dk, dv, lens", LINEAR_CASES)
 @pytest.mark.parametrize("rank", [1, 16, 37])
-def test_gated_linear_attention_kernel(heads, dk, dv, lens, rank):
-    """Decays from a projection of low rank and the recurrence, whole and in every cutting, against the plain functions."""
+@pytest.mark.parametrize("in_chunks", [False, True])
+def test_gated_linear_attention_kernel(heads, dk, dv, lens, rank, in_chunks):
+    """Decays from a projection of low rank and the recurrence, whole and in every cutting, token by token and (longer portions)
+    in chunks, against the plain functions."""
     torch.manual_seed(dk + dv + rank)
     H, n, tau, scale = heads, sum(lens), 5.0, 0.3
     low_off = 3 + 2 * H * dk + H * dv
@@ -110,17 +118,19 @@ def test_gated_linear_attention_kernel(heads, dk, dv, lens, rank):
         at += ln
     want = torch.cat(want).float()
     ops_args = (up.cuda(), bias.cuda(), tau, scale)
-    for steps in cuts_of(lens, True):
+    for steps in cuts_of(lens):
         state = torch.zeros(len(lens) + 1, ops.linear_attention_state_words(H, dk, dv), device="cuda")
-        (o,) = walk(lambda rows, qs, sl, pos, longest: (ops.gated_linear_attention(
-            rows, 3, 3 + H * dk, 3 + 2 * H * dk, low_off, *ops_args, state, qs, sl, H, dk, dv, longest=longest),), proj, lens, slots, steps)
+        (o,) = walk(lambda rows, qs, sl, pos, longest, chunks: (ops.gated_linear_attention(
+            rows, 3, 3 + H * dk, 3 + 2 * H * dk, low_off, *ops_args, state, qs, sl, H, dk, dv, longest=longest,
+            chunks=chunks),), proj, lens, slots, steps, in_chunks)
         torch.testing.assert_close(o, want, atol=2e-4, rtol=2e-4)
         assert float(state[len(lens)].abs().max()) == 0.0  # nobody's slot
 
 
 @pytest.mark.parametrize("heads, dk, dv, lens", LINEAR_CASES + [(2, 8, 8, [1100, 513]), (1, 24, 16, [512, 511, 1])])
 @pytest.mark.parametrize("sharp", [False, True])
-def test_matrix_memory_kernel(heads, dk, dv, lens, sharp):
+@pytest.mark.parametrize("in_chunks", [False, True])
+def test_matrix_memory_kernel(heads, dk, dv, lens, sharp, in_chunks):
     """Gates, the running maximum, the state and its read-out, whole and in every cutting, against the plain function;
     ``sharp``: gates near their caps, so that the maximum jumps and falls."""
     torch.manual_seed(dk + dv)
@@ -133,25 +143,33 @@ def test_matrix_memory_kernel(heads, dk, dv, lens, sharp):
         proj[:, f_off : f_off + H] *= 6.0
     i_bias, f_bias = torch.randn(H), torch.randn(H) + 2.0
     slots = list(range(len(lens)))[::-1]
-    want, at = [], 0
+    # the read-outs of S and n, and the maxima, apart: their quotient is the plain function's
+    sums, keys, tops, at = [], [], [], 0
     for ln in lens:
         p = proj[at : at + ln].double()
         q, k, v = (p[:, o : o + H * w].reshape(ln, H, w) for o, w in ((2, dk), (2 + H * dk, dk), (2 + 2 * H * dk, dv)))
         i = pt.soft_cap(p[:, i_off : i_off + H] + i_bias.double(), cap)
         f = pt.log_sigmoid(pt.soft_cap(p[:, f_off : f_off + H] + f_bias.double(), cap))
-        want.append(pt.matrix_memory(q * scale, k, v, i, f).reshape(ln, H * dv))
+        m = torch.zeros(ln + 1, H, dtype=torch.float64)
+        for t in range(ln):
+            m[t + 1] = torch.maximum(f[t] + m[t], i[t])
+        keep, write = torch.exp(f + m[:-1] - m[1:])[..., None].expand(ln, H, dk), torch.exp(i - m[1:])[..., None]
+        sums.append(pt.decayed_outer_products(q * scale, k * write, v, keep))
+        keys.append(pt.decayed_outer_products(q * scale, k * write, torch.ones(ln, H, 1, dtype=torch.float64), keep)[..., 0])
+        tops.append(m[1:])
+        whole = sums[-1] / (torch.maximum(keys[-1].abs(), torch.exp(-m[1:])) + 1e-6)[..., None]
+        assert torch.allclose(whole, pt.matrix_memory(q * scale, k, v, i, f))
         at += ln
-    want = torch.cat(want)
-    for steps in cuts_of(lens, True):
+    want = torch.cat([torch.cat(sums), torch.cat(keys)[..., None]], dim=-1)
+    size = want.abs().amax(-1, keepdim=True).amax(1, keepdim=True) + 0.1
+    for steps in cuts_of(lens):
         state = torch.zeros(len(lens) + 1, ops.linear_attention_state_words(H, dk, dv, memory=True), device="cuda")
-        o, floor = walk(lambda rows, qs, sl, pos, longest: ops.matrix_memory(
+        o, floor = walk(lambda rows, qs, sl, pos, longest, chunks: ops.matrix_memory(
             rows, 2, 2 + H * dk, 2 + 2 * H * dk, i_off, f_off, i_bias.cuda(), f_bias.cuda(), cap, scale, state, qs, sl, pos, H, dk, dv,
-            longest=longest), proj, lens, slots, steps)
+            longest=longest, chunks=chunks), proj, lens, slots, steps, in_chunks)
         o = o.view(n, H, -1).double()
-        got = o[..., :dv] / (torch.maximum(o[..., dv].abs(), floor.double()) + 1e-6)[..., None]
-        # (where n . q nearly cancels, the quotient magnifies the sums' rounding: compare by the row's own size)
-        err = (got.reshape(n, H * dv) - want).abs() / (want.abs().amax(1, keepdim=True) + 1e-2)
-        assert float(err.max()) < 2e-3 and float(err.median()) < 1e-5
+        assert float(((o[..., : dv + 1] - want).abs() / size).max()) < 1e-4
+        torch.testing.assert_close(floor.double(), torch.exp(-torch.cat(tops)), atol=1e-7, rtol=1e-4)
         assert float(state[len(lens)].abs().max()) == 0.0
 
 

@@ -22,47 +22,14 @@
 // do not meet: a column is owned by LA_LANES neighbouring lanes that cut dk between them and add up through the
 // wavefront's own data paths, always in the same order, so a token's result does not depend on how its request's
 // tokens were cut into steps or on what shares the batch (the running maxima of a portion are combined in an order of
-// its own: they change a result by rounding only).
-#include "common.h"
+// its own: they change a result by rounding only).  Longer portions of the last two forms go in chunks of products on the
+// matrix cores instead, with the same 32-bit sums in another order: linear_attention_chunks.hip.
+#include "linear_attention.h"
 
 #define LA_LANES 16
 #define LA_COLS 4      // columns a wavefront owns
 #define LA_WAVES 8     // most wavefronts of a workgroup (they share nothing: a workgroup is only a unit of dispatch)
-enum { LA_CONSTANT = 0, LA_FORGET = 1, LA_CHANNEL = 2, LA_MEMORY = 3 };
 
-// The arguments of one call; the same fields in the same order in kernels/ops.py.
-struct LaArgs {
-  const float* proj;
-  int ld, q_off, k_off, v_off;
-  const float* decay;              // LA_CONSTANT [H]
-  const float *forget_bias, *forget_low;  // LA_FORGET [H * dk]
-  int low_off, rank;               // LA_CHANNEL: the low-rank sums' first column and number
-  const float *low_up, *low_bias;  // [rank][H * dk], [H * dk]
-  float tau;
-  int i_off, f_off;                // LA_MEMORY: first columns of the gates' sums
-  const float *i_bias, *f_bias;    // [H]
-  float cap, q_scale;
-  float* state;
-  size_t state_stride;
-  const int *q_start, *slots, *positions;
-  float* rec;    // working memory of steps with longer portions: tk_linear_attention_work_words 32-bit words a token
-  float* o;      // [tokens][H][o_head]
-  float* floor;  // LA_MEMORY [tokens][H]
-  int o_head;
-  int n_tokens, n_requests, H, dk, dv, longest;
-};
-
-__device__ __forceinline__ float la_silu(float x) { return x / (1.0f + expf(-x)); }
-__device__ __forceinline__ float la_sigmoid(float x) { return 1.0f / (1.0f + expf(-x)); }
-// the forget gate, written out in one multiply-add so that every kernel that computes it gets the same bits
-__device__ __forceinline__ float la_forget(float x, float bias, float lo) { return fmaf(1.0f - lo, la_sigmoid(x + bias), lo); }
-__device__ __forceinline__ float la_log_sigmoid(float x) { return fminf(x, 0.f) - log1pf(expf(-fabsf(x))); }
-__device__ __forceinline__ float la_channel_decay(float z, float tau) { return expf(la_log_sigmoid(z) / tau); }
-__device__ __forceinline__ float la_soft_cap(float x, float cap) { return cap * tanhf(x / cap); }
-
-// columns of a head's state: the values', and the keys' sum in the last form
-template <int MODE>
-__host__ __device__ __forceinline__ int la_columns(int dv) { return MODE == LA_MEMORY ? dv + 1 : dv; }
 // A row of `rec`: [q: H x dkp | k or f: H x dkp | (LA_CHANNEL) a: H x dkp | v: H x columns, padded to a multiple of 4],
 // dkp = dk rounded up to 64 times the pieces a lane holds, zeros in the padding (a padded row of S meets a zero of q).
 template <int MODE>
@@ -71,11 +38,6 @@ template <int MODE>
 __host__ __device__ __forceinline__ int la_rec_width(int H, int dkp, int dv) {
   return la_value_at<MODE>(H, dkp) + (H * la_columns<MODE>(dv) + 3) / 4 * 4;
 }
-// where the running maximum after position p of head h is kept
-__device__ __forceinline__ size_t la_max_at(const LaArgs& a, int p, int h) {
-  return (size_t)a.H * (a.dv + 1) * a.dk + (size_t)(p & 1) * a.H + h;
-}
-
 // --------------------------------------------------------------------------
 // Before the recurrence, once a token: the activations, into rows that the recurrence's lanes read 16 bytes at a time
 // (LA_CHANNEL: without the decays).
@@ -442,6 +404,10 @@ TK_API int tk_linear_attention_work_words(int mode, int H, int dk, int dv, int l
   return mode == LA_CHANNEL ? la_rec_width<LA_CHANNEL>(H, dkp, dv) : la_rec_width<LA_CONSTANT>(H, dkp, dv);
 }
 
+void la_launch_gates(const LaArgs& a, float2* gates, int log_decay, hipStream_t stream) {
+  hipLaunchKernelGGL(linear_attention_gates_kernel, dim3(a.H, a.n_requests), dim3(LA_GATES), 0, stream, a, gates, log_decay);
+}
+
 template <int MODE>
 static int la_run(const LaArgs& a, hipStream_t stream) {
   const int columns = la_columns<MODE>(a.dv), all_waves = (columns + LA_COLS - 1) / LA_COLS;
@@ -469,7 +435,7 @@ static int la_run(const LaArgs& a, hipStream_t stream) {
                        0, stream, a, dkp);
   if (MODE == LA_MEMORY) {
     gates = (float2*)(a.rec + (size_t)a.n_tokens * ld_rec);  // (rows are multiples of 16 bytes)
-    hipLaunchKernelGGL(linear_attention_gates_kernel, dim3(a.H, a.n_requests), dim3(LA_GATES), 0, stream, a, gates, 0);
+    la_launch_gates(a, gates, 0, stream);
   }
   // A long walk is a chain of arithmetic in every wavefront: one wavefront a workgroup then spreads a prompt's few
   // wavefronts over all compute units (measured: 2 048 tokens of 8 heads of 128 x 128 in 180 us, against 360 us with
@@ -510,7 +476,10 @@ TK_API int tk_linear_attention(int mode, const LaArgs* args, hipStream_t stream)
              "linear_attention: a pointer is missing, the state's or the result's rows are too short or the step too large");
   TK_REQUIRE((((uintptr_t)a.rec | (uintptr_t)a.state) & 15) == 0, "linear_attention: rec and state must start at multiples of 16 bytes");
   TK_REQUIRE(a.longest >= 1, "linear_attention: the longest portion of a step with tokens is at least one token");
+  TK_REQUIRE(a.n_chunks == 0 || (a.n_chunks > 0 && a.chunk_req && a.chunk_row0 && a.first_chunk && la_chunks_take(mode, a.dk, a.longest)),
+             "linear_attention: the chunked form does not take these sizes, or its plan is missing");
   if (a.n_requests == 0 || a.n_tokens == 0) return 0;
+  if (a.n_chunks > 0) return la_run_chunks(mode, a, stream);
   switch (mode) {
     case LA_CONSTANT: return la_run<LA_CONSTANT>(a, stream);
     case LA_FORGET: return la_run<LA_FORGET>(a, stream);

@@ -43,6 +43,8 @@ _SIGNATURES: dict[str, dict[str, list]] = {
         "tk_linear_attention": [c_int, _P, _P],
         "tk_linear_attention_state_words": [c_int] * 4,
         "tk_linear_attention_work_words": [c_int] * 5,
+        "tk_linear_attention_chunk_words": [c_int] * 4,
+        "tk_linear_attention_chunk_tokens": [],
         "tk_group_norm_gate": [c_int, _P, c_int, _P, c_int, c_int, _P, c_int, _P, c_float, c_float, _P, c_int, c_int, c_int, c_int, _P],
         "tk_sigmoid_gate": [c_int, _P, c_int, _P, c_int, c_float, _P, c_int, c_int, c_int, _P],
         "tk_short_conv": [c_int, _P, c_int, _P, c_int, _P, c_size_t, _P, _P, _P, _P] + [c_int] * 4 + [_P],

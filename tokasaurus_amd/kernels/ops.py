@@ -1244,6 +1244,7 @@ class _LinearAttentionArgs(ctypes.Structure):
         ("q_start", ctypes.c_void_p), ("slots", ctypes.c_void_p), ("positions", ctypes.c_void_p), ("rec", ctypes.c_void_p),
         ("o", ctypes.c_void_p), ("floor", ctypes.c_void_p), ("o_head", ctypes.c_int), ("n_tokens", ctypes.c_int),
         ("n_requests", ctypes.c_int), ("H", ctypes.c_int), ("dk", ctypes.c_int), ("dv", ctypes.c_int), ("longest", ctypes.c_int),
+        ("chunk_req", ctypes.c_void_p), ("chunk_row0", ctypes.c_void_p), ("first_chunk", ctypes.c_void_p), ("n_chunks", ctypes.c_int),
     ]
 
 
@@ -1257,9 +1258,28 @@ def linear_attention_state_words(heads: int, key_dim: int, value_dim: int, memor
     return heads * value_dim * key_dim
 
 
+@dataclass
+class ChunkPlan:
+    """A step's rows cut into chunks of ``linear_attention_chunk_tokens`` neighbouring tokens of one request, in the requests'
+    order: every chunk's request and first row, and every request's first chunk (and, last, the number of chunks), int32."""
+
+    req: torch.Tensor
+    row0: torch.Tensor
+    first: torch.Tensor
+
+
+def linear_attention_chunk_tokens() -> int:
+    return load("core").tk_linear_attention_chunk_tokens()
+
+
+def linear_attention_takes_chunks(memory: bool, key_dim: int, longest: int) -> bool:
+    """Whether a step whose longest portion has this many tokens goes in chunks (and so needs a ``ChunkPlan``)."""
+    return load("core").tk_linear_attention_chunk_words(LA_MEMORY if memory else LA_CHANNEL, 1, int(key_dim), int(longest)) > 0
+
+
 def _linear_attention(mode: int, proj: torch.Tensor, q_off: int, k_off: int, v_off: int, state: torch.Tensor, q_start: torch.Tensor,
                       slots: torch.Tensor, heads: int, key_dim: int, value_dim: int, longest: int | None, extra: dict,
-                      o_head: int | None = None) -> torch.Tensor:
+                      o_head: int | None = None, chunks: ChunkPlan | None = None) -> torch.Tensor:
     """What the forms of the recurrence share: checks, working memory, the result [tokens, heads * o_head]."""
     _gpu(proj, state, q_start, slots)
     _need(proj.dim() == 2 and proj.dtype == torch.float32 and proj.stride(1) == 1, "linear_attention: 32-bit rows with unit inner stride")
@@ -1280,8 +1300,22 @@ def _linear_attention(mode: int, proj: torch.Tensor, q_off: int, k_off: int, v_o
         longest = max(1, int(n if longest is None else longest))
         # the activated rows that the recurrence reads: passes over the step's tokens in front of it (a step of single
         # tokens computes them in the recurrence's own kernel)
-        work = load("core").tk_linear_attention_work_words(mode, H, dk, dv, longest)
-        rec = torch.empty((n, work), dtype=torch.float32, device=proj.device) if work else None
+        n_chunks, chunk_words = 0, 0
+        if chunks is not None:
+            chunk_words = load("core").tk_linear_attention_chunk_words(mode, H, dk, longest)
+        if chunk_words:
+            _gpu(chunks.req, chunks.row0, chunks.first)
+            for t, name in ((chunks.req, "chunk requests"), (chunks.row0, "chunk rows"), (chunks.first, "first chunks")):
+                _i32(t, name)
+            n_chunks = chunks.req.numel()
+            _need(n_chunks > 0 and chunks.row0.numel() == n_chunks and chunks.first.numel() == slots.numel() + 1,
+                  "linear_attention: one request and one row a chunk, one first chunk a request")
+            extra = dict(extra, chunk_req=chunks.req.data_ptr(), chunk_row0=chunks.row0.data_ptr(), first_chunk=chunks.first.data_ptr(),
+                         n_chunks=n_chunks)
+            work = n_chunks * chunk_words + (2 * n * H if mode == LA_MEMORY else 0)
+        else:
+            work = n * load("core").tk_linear_attention_work_words(mode, H, dk, dv, longest)
+        rec = torch.empty((work,), dtype=torch.float32, device=proj.device) if work else None
         a = _LinearAttentionArgs(proj=proj.data_ptr(), ld=proj.stride(0), q_off=int(q_off), k_off=int(k_off), v_off=int(v_off),
                                  state=state.data_ptr(), state_stride=state.stride(0), q_start=q_start.data_ptr(), slots=slots.data_ptr(),
                                  rec=rec.data_ptr() if rec is not None else None, o=o.data_ptr(), o_head=o_head, n_tokens=n,
@@ -1315,10 +1349,12 @@ def linear_attention(proj: torch.Tensor, q_off: int, k_off: int, v_off: int, sta
 
 def gated_linear_attention(proj: torch.Tensor, q_off: int, k_off: int, v_off: int, low_off: int, low_up: torch.Tensor,
                            low_bias: torch.Tensor, tau: float, q_scale: float, state: torch.Tensor, q_start: torch.Tensor,
-                           slots: torch.Tensor, heads: int, key_dim: int, value_dim: int, longest: int | None = None) -> torch.Tensor:
+                           slots: torch.Tensor, heads: int, key_dim: int, value_dim: int, longest: int | None = None,
+                           chunks: ChunkPlan | None = None) -> torch.Tensor:
     """The recurrence of ``linear_attention`` with q (times ``q_scale``), k and v as they are and a decay per head and key
     channel, ``a = sigmoid(z)^(1 / tau)`` with ``z = low_up^T low + low_bias``: ``low`` are the sums from column ``low_off``
-    on, ``low_up`` [rank, heads * key_dim] and ``low_bias`` are 32-bit."""
+    on, ``low_up`` [rank, heads * key_dim] and ``low_bias`` are 32-bit.  ``chunks``: longer portions go in chunks on the matrix
+    cores (where ``linear_attention_takes_chunks``; 32-bit products, the sums in another order)."""
     _gpu(low_up, low_bias)
     _need(low_up.dim() == 2 and low_up.shape[1] == heads * key_dim and low_up.dtype == torch.float32 and low_up.is_contiguous(),
           "gated_linear_attention: the low-rank projection's second matrix must be contiguous float32 [rank, heads * key_dim]")
@@ -1327,18 +1363,19 @@ def gated_linear_attention(proj: torch.Tensor, q_off: int, k_off: int, v_off: in
     _need(0 <= low_off and low_off + rank <= proj.shape[1], "gated_linear_attention: the low-rank sums lie outside the rows")
     return _linear_attention(LA_CHANNEL, proj, q_off, k_off, v_off, state, q_start, slots, heads, key_dim, value_dim, longest,
                              dict(low_off=int(low_off), rank=rank, low_up=low_up.data_ptr(), low_bias=low_bias.data_ptr(), tau=float(tau),
-                                  q_scale=float(q_scale)))
+                                  q_scale=float(q_scale)), chunks=chunks)
 
 
 def matrix_memory(proj: torch.Tensor, q_off: int, k_off: int, v_off: int, i_off: int, f_off: int, i_bias: torch.Tensor,
                   f_bias: torch.Tensor, cap: float, q_scale: float, state: torch.Tensor, q_start: torch.Tensor, slots: torch.Tensor,
-                  positions: torch.Tensor, heads: int, key_dim: int, value_dim: int, longest: int | None = None
-                  ) -> tuple[torch.Tensor, torch.Tensor]:
+                  positions: torch.Tensor, heads: int, key_dim: int, value_dim: int, longest: int | None = None,
+                  chunks: ChunkPlan | None = None) -> tuple[torch.Tensor, torch.Tensor]:
     """The matrix memory of xLSTM (mLSTM) from the 32-bit sums ``proj``: q (times ``q_scale``), k and v as they are; per head
     and token the log gates ``i = cap tanh((. + i_bias) / cap)`` and ``f = log sigmoid(cap tanh((. + f_bias) / cap))`` (sums
     from ``i_off`` and ``f_off`` on); with the running maximum ``m' = max(f + m, i)``, ``S <- exp(f + m - m') S + exp(i - m')
     k v^T`` and n likewise with k alone.  Returns what ``group_norm_gate`` takes as ``o`` and ``floor``: [tokens, heads * w]
-    with ``S^T q`` of a head and, behind it, ``n . q`` (w: value_dim + 1 rounded up to a multiple of 4), and exp(-m') [tokens, heads]."""
+    with ``S^T q`` of a head and, behind it, ``n . q`` (w: value_dim + 1 rounded up to a multiple of 4), and exp(-m') [tokens, heads].
+    ``chunks`` as in ``gated_linear_attention``."""
     _gpu(i_bias, f_bias, positions)
     _i32(positions, "positions")
     _need(positions.numel() == proj.shape[0], "matrix_memory: one position a token")
@@ -1350,7 +1387,7 @@ def matrix_memory(proj: torch.Tensor, q_off: int, k_off: int, v_off: int, i_off:
     o = _linear_attention(LA_MEMORY, proj, q_off, k_off, v_off, state, q_start, slots, heads, key_dim, value_dim, longest,
                           dict(i_off=int(i_off), f_off=int(f_off), i_bias=i_bias.data_ptr(), f_bias=f_bias.data_ptr(), cap=float(cap),
                                q_scale=float(q_scale), positions=positions.data_ptr(), floor=floor.data_ptr()),
-                          o_head=-(-(value_dim + 1) // 4) * 4)
+                          o_head=-(-(value_dim + 1) // 4) * 4, chunks=chunks)
     return o, floor
 
 

@@ -32,8 +32,27 @@ from __future__ import annotations
 import torch
 
 from tokasaurus_amd.kernels import ops
+from tokasaurus_amd.kernels.upload import upload
 from tokasaurus_amd.parts.base import BIAS, MATRIX, MIXERS, NORM_WEIGHT, UNIT_INTERVAL, VECTOR, Mixer, StateNeed, StepContext, TensorSpec
 from tokasaurus_amd.parts.linear import Linear, Placer
+
+
+def chunk_plan(ctx: StepContext, memory: bool, key_dim: int) -> "ops.ChunkPlan | None":
+    """The step's rows in chunks, made once a step and shared by the layers; None for steps of short portions."""
+    if not ops.linear_attention_takes_chunks(memory, key_dim, ctx.max_q_len):
+        return None
+    plan = ctx.extras.get("chunk_plan")
+    if plan is None:
+        size = ops.linear_attention_chunk_tokens()
+        req, row0, first = [], [], [0]
+        for r in range(ctx.num_requests):
+            rows = range(ctx.host_q_start[r], ctx.host_q_start[r + 1], size)
+            req += [r] * len(rows)
+            row0 += rows
+            first.append(len(req))
+        dev, n = upload(req + row0 + first, torch.int32, ctx.device), len(req)
+        plan = ctx.extras["chunk_plan"] = ops.ChunkPlan(dev[:n], dev[n : 2 * n], dev[2 * n :])
+    return plan
 
 
 class _LinearAttention(Mixer):
@@ -184,7 +203,8 @@ class GatedLinearAttention(_LinearAttention):
         qk, v = H * dk, H * dv
         proj = self.inp(h, out_f32=True)
         o = ops.gated_linear_attention(proj, 0, qk, 2 * qk, 2 * (qk + v), self.low_up, self.low_bias, self.tau, self.q_scale, state,
-                                       ctx.q_start, ctx.slots, H, dk, dv, longest=ctx.max_q_len)
+                                       ctx.q_start, ctx.slots, H, dk, dv, longest=ctx.max_q_len,
+                                       chunks=chunk_plan(ctx, False, dk))
         return ops.group_norm_gate(o, self.norm_w, self.norm_eps, H, h.dtype, gate=proj[:, 2 * qk + v : 2 * (qk + v)], scale=scale, out=out,
                                    silu_gate=True)
 
@@ -229,6 +249,7 @@ class MatrixMemory(_LinearAttention):
         qk, v = H * dk, H * dv
         proj = self.inp(h, out_f32=True)
         o, floor = ops.matrix_memory(proj, 0, qk, 2 * qk, 2 * (qk + v), 2 * (qk + v) + H, self.i_bias, self.f_bias, self.gate_cap,
-                                     self.q_scale, state, ctx.q_start, ctx.slots, ctx.positions, H, dk, dv, longest=ctx.max_q_len)
+                                     self.q_scale, state, ctx.q_start, ctx.slots, ctx.positions, H, dk, dv, longest=ctx.max_q_len,
+                                     chunks=chunk_plan(ctx, True, dk))
         return ops.group_norm_gate(o, self.norm_w, self.norm_eps, H, h.dtype, gate=proj[:, 2 * qk + v : 2 * (qk + v)], scale=scale, out=out,
                                    size=dv, floor=floor)
