@@ -348,6 +348,24 @@ def test_every_cutting_gives_the_plain_rows(tefavik_folders, name, dtype):
             assert float((a[key] - b[key]).abs().max()) < 2e-4 * max(1.0, float(a[key].abs().max()))
 
 
+@pytest.mark.parametrize("name", ["mixed", "large_heads"])
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+def test_long_prompts_in_one_step(tefavik_folders, name, dtype):
+    """Steps of hundreds of rows, in which the two mixers of a layer run at the same time, one after the other and the same
+    step again: every row is the plain one's, and the steps' rows are equal bit for bit."""
+    folder, vocab = tefavik_folders[name], CONFIGS[name]["vocab"]
+    reqs = {f"l{i}": random_tokens(n, vocab, 60 + i) for i, n in enumerate((230, 20, 131))}
+    plain = plain_rows(folder, reqs)
+    limits = rounding_limits(folder, reqs) if dtype == "bfloat16" else None
+    runner = runner_for(folder, dtype, tokens=512)
+    steps = [{"entries": [(rid, toks, list(range(len(toks)))) for rid, toks in reqs.items()], "end": list(reqs)}]
+    first = run_steps(runner, steps)
+    compare_rows(first, plain, TOL[dtype], limits)
+    for _ in range(3):
+        again = run_steps(runner, steps)
+        assert all(torch.equal(again[key], row) for key, row in first.items())
+
+
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
 def test_only_the_last_row_is_wanted(tefavik_folders, dtype):
     """The last block goes on with the wanted rows alone: their experts are their own tokens'."""

@@ -78,15 +78,6 @@ __global__ __launch_bounds__(256) void linear_attention_prepare_kernel(LaArgs a,
   a.rec[t * ld_rec + x] = val;
 }
 
-// z of channel c: the second matrix of the low-rank projection on `low` (the order of the sum is the same everywhere)
-__device__ __forceinline__ float la_low_rank(const LaArgs& a, const float* low, int c) {
-  float z = 0.f;
-  const int width = a.H * a.dk;
-#pragma unroll 8
-  for (int r = 0; r < a.rank; ++r) z = fmaf(low[r], a.low_up[(size_t)r * width + c], z);
-  return z + a.low_bias[c];
-}
-
 // The decays of LA_CHANNEL into `rec`: a thread one channel of LA_TOKENS neighbouring tokens, which share the loads of
 // the second matrix.
 #define LA_TOKENS 8
@@ -289,13 +280,14 @@ static int la_pieces(int dk) {
 
 // --------------------------------------------------------------------------
 // The same for steps in which every request brings one token: the activations are computed by the lanes that need
-// them (there is no pass in front and no `rec`), with the functions of the pass above, so the sums are the same bits.
-// LA_CHANNEL: a workgroup computes its head's decays into LDS.  LA_MEMORY: every lane computes its head's two gates.
+// them (there is no pass in front and no `rec`), with the functions of the pass above, so the sums are the same bits (up to
+// the order of LA_CHANNEL's low-rank sums: a workgroup computes its head's decays into LDS).  LA_MEMORY: every lane computes its head's two gates.
 // --------------------------------------------------------------------------
 template <int NQ, int MODE>
 __global__ __launch_bounds__(LA_WAVES * TK_WAVE) void linear_attention_single_kernel(LaArgs a, const float* __restrict__ proj,
                                                                                  float* __restrict__ o) {
-  __shared__ __align__(16) float decays[MODE == LA_CHANNEL ? NQ * 64 : 4];
+  constexpr int PARTS = 4;  // the low-rank sums of a channel are cut among so many threads where the workgroup has them
+  __shared__ __align__(16) float decays[MODE == LA_CHANNEL ? NQ * 64 : 4], part[MODE == LA_CHANNEL ? PARTS * NQ * 64 : 4];
   const int h = blockIdx.x, r = blockIdx.y;
   const int lane = threadIdx.x % LA_LANES, grp = threadIdx.x / LA_LANES;
   const int dk = a.dk, columns = la_columns<MODE>(a.dv);
@@ -321,8 +313,22 @@ __global__ __launch_bounds__(LA_WAVES * TK_WAVE) void linear_attention_single_ke
     }
   }
   if (MODE == LA_CHANNEL) {
-    for (int i = threadIdx.x; i < NQ * 64; i += blockDim.x)
-      decays[i] = i < dk ? la_channel_decay(la_low_rank(a, row + a.low_off, h * dk + i), a.tau) : 0.f;
+    const int parts = min(PARTS, max(1, (int)blockDim.x / (NQ * 64))), width = a.H * dk;
+    for (int x = threadIdx.x; x < parts * NQ * 64; x += blockDim.x) {
+      const int i = x % (NQ * 64);
+      float z = 0.f;
+      if (i < dk) {
+#pragma unroll 8
+        for (int r = x / (NQ * 64); r < a.rank; r += parts) z = fmaf(row[a.low_off + r], a.low_up[(size_t)r * width + h * dk + i], z);
+      }
+      part[x] = z;
+    }
+    __syncthreads();
+    for (int i = threadIdx.x; i < NQ * 64; i += blockDim.x) {
+      float z = 0.f;
+      for (int k = 0; k < parts; ++k) z += part[k * NQ * 64 + i];
+      decays[i] = i < dk ? la_channel_decay(z + a.low_bias[h * dk + i], a.tau) : 0.f;
+    }
     __syncthreads();
   }
   float keep = MODE == LA_CONSTANT ? a.decay[h] : 0.f;

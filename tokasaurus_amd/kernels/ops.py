@@ -12,6 +12,7 @@ from dataclasses import dataclass
 
 import torch
 
+from tokasaurus_amd.kernels import lanes
 from tokasaurus_amd.kernels.library import KernelError, call, load
 
 _DT = {torch.float32: 0, torch.bfloat16: 1}
@@ -1057,16 +1058,18 @@ def add(x: torch.Tensor, y: torch.Tensor) -> torch.Tensor:
 # What the product library's kernels may use for partial sums: its stream-K kernels want up to 64 MB
 # (one 256 x 256 tile of 32-bit sums a compute unit); the tensor library gives its products 76 MB too.
 LIBRARY_WORKSPACE_BYTES = 76 << 20
-_library_workspace: dict[int, torch.Tensor] = {}
+_library_workspace: dict[tuple[int, int], torch.Tensor] = {}
 
 
 def library_workspace() -> torch.Tensor:
     """The current device's workspace for library products: made at the first call (a runner
-    makes it before it records steps, so that no recording allocates it) and kept."""
+    makes it before it records steps, so that no recording allocates it) and kept; one a lane
+    (``kernels.lanes``), for calls that run at the same time."""
     device = torch._C._cuda_getDevice()
-    ws = _library_workspace.get(device)
+    key = (device, lanes.lane())
+    ws = _library_workspace.get(key)
     if ws is None:
-        ws = _library_workspace[device] = torch.empty(LIBRARY_WORKSPACE_BYTES, dtype=torch.uint8, device=f"cuda:{device}")
+        ws = _library_workspace[key] = torch.empty(LIBRARY_WORKSPACE_BYTES, dtype=torch.uint8, device=f"cuda:{device}")
     return ws
 
 

@@ -6,7 +6,7 @@ the matrices side by side, ``[W_o left | W_o right]``, whose 32-bit sums are the
 mixers' results.  Or (``out_norms``) each mixer's own output, the full width, passes an RMS norm with a plain weight
 before the two are summed: ``left_scale * (rms_norm(left(h)) * w_left + rms_norm(right(h)) * w_right)``, both scales being
 equal; the two output projections are then products of their own, whose 32-bit sums a block may norm, sum and add to its
-stream in one pass (``normed_sum``).  At most one of the two keeps keys in pages and at most one a state in the request's slot.
+stream in one pass (``normed_sum``), and in steps of many rows the two mixers run at the same time.  At most one of the two keeps keys in pages and at most one a state in the request's slot.
 """
 
 from __future__ import annotations
@@ -14,8 +14,12 @@ from __future__ import annotations
 import torch
 
 from tokasaurus_amd.kernels import ops
+from tokasaurus_amd.kernels.lanes import beside, join
 from tokasaurus_amd.parts.base import MIXERS, NORM_WEIGHT, CacheNeed, Mixer, NormedSum, Part, PartSpec, StateNeed, TensorSpec
 from tokasaurus_amd.parts.linear import Linear, Placer
+
+
+BESIDE_FROM_ROWS = 256
 
 
 @MIXERS.register("mixer_pair")
@@ -81,11 +85,20 @@ class MixerPair(Mixer):
         return both if rows is None else ops.gather_rows(both, rows)
 
     def normed_sum(self, h, ctx, cache, state, rows) -> NormedSum:
-        outs = []
-        for m in (self.left, self.right):
+        def branch(m):
             y = m.inner_rows(h, ctx, cache if m.cache_need() is not None else None, state if m.state_need() is not None else None)
-            outs.append(m.out(y if rows is None else ops.gather_rows(y, rows), out_f32=True))
-        return NormedSum(outs[0], self.norm_w[0], outs[1], self.norm_w[1], float(self.out_norms["eps"]), self.left_scale)
+            return m.out(y if rows is None else ops.gather_rows(y, rows), out_f32=True)
+
+        # steps of many rows: the two at the same time, for neither fills the chip (a recurrence is few long walks).  Recorded
+        # steps are left in one line: there the branches' hand-overs cost what they save.
+        if h.shape[0] >= BESIDE_FROM_ROWS and not ctx.extras.get("static"):
+            with beside():
+                right = branch(self.right)
+            left = branch(self.left)
+            join()
+        else:
+            left, right = branch(self.left), branch(self.right)
+        return NormedSum(left, self.norm_w[0], right, self.norm_w[1], float(self.out_norms["eps"]), self.left_scale)
 
     def mix(self, h, ctx, cache, state, rows, out_f32: bool = False):
         if self.out_norms:
