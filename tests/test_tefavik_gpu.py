@@ -351,8 +351,8 @@ def test_every_cutting_gives_the_plain_rows(tefavik_folders, name, dtype):
 @pytest.mark.parametrize("name", ["mixed", "large_heads"])
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
 def test_long_prompts_in_one_step(tefavik_folders, name, dtype):
-    """Steps of hundreds of rows, in which the two mixers of a layer run at the same time, one after the other and the same
-    step again: every row is the plain one's, and the steps' rows are equal bit for bit."""
+    """Steps of hundreds of rows, the same step again and again: every row is the plain one's, and the steps' rows are equal
+    bit for bit."""
     folder, vocab = tefavik_folders[name], CONFIGS[name]["vocab"]
     reqs = {f"l{i}": random_tokens(n, vocab, 60 + i) for i, n in enumerate((230, 20, 131))}
     plain = plain_rows(folder, reqs)

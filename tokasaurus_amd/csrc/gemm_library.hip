@@ -8,7 +8,8 @@
 // The kernel chosen is the one the tensor library's own product gets from the same question.
 //
 // No device memory is allocated here: the caller brings the workspace that the library's
-// kernels may use (stream-K partial sums), the same for every call on a stream.
+// kernels may use (stream-K partial sums), the same for every call on a stream.  A device's calls are to be on one stream at
+// a time: they share a handle, and a stream-K kernel's workgroups wait for one another.
 #include "common.h"
 
 #include <hipblaslt/hipblaslt.h>

@@ -312,16 +312,30 @@ TK_API int tk_grouped_gemm_bf16(const void* A, int lda, const int* a_row, const 
 }
 
 // --------------------------------------------------------------------------
-// Pairs (token, place) -> slots sorted by expert.  One workgroup.  Expert e's pairs take the slots
+// Pairs (token, place) -> slots sorted by expert.  A workgroup a job: a layer's choice, or (where the choice of several layers
+// is known before the first of them runs) all layers' in one launch.  Expert e's pairs take the slots
 // first[e] .. first[e] + count[e] - 1 with first[e] a multiple of tm; the slots between a run's end and the
 // next multiple are empty.  slot_pair[slot] = the pair (or -1), slot_token[slot] = its token (or -1),
 // tile_group[tile] = the expert whose run the tile lies in (or -1), tile_group[max_tiles] = the tiles in use.  Pairs of identity experts (ids >= experts)
 // and empty places (ids < 0) get no slot.  Which of an expert's slots a pair gets depends on the order of
 // arrival and changes no result: every row is computed on its own.
 // --------------------------------------------------------------------------
-__global__ __launch_bounds__(1024) void expert_sort_kernel(const int* __restrict__ ids, int pairs, int top, int experts,
-                                                           int max_tiles, int tm, int* __restrict__ slot_pair,
-                                                           int* __restrict__ slot_token, int* __restrict__ tile_group) {
+struct SortJob {
+  const int* ids;
+  int *slot_pair, *slot_token, *tile_group;
+  int pairs, top, experts, max_tiles, tm;
+};
+#define SORT_JOBS 48
+struct SortJobs {
+  SortJob job[SORT_JOBS];
+};
+__global__ __launch_bounds__(1024) void expert_sort_kernel(SortJobs jobs) {
+  const SortJob& jb = jobs.job[blockIdx.x];
+  const int* __restrict__ ids = jb.ids;
+  const int pairs = jb.pairs, top = jb.top, experts = jb.experts, max_tiles = jb.max_tiles, tm = jb.tm;
+  int* __restrict__ slot_pair = jb.slot_pair;
+  int* __restrict__ slot_token = jb.slot_token;
+  int* __restrict__ tile_group = jb.tile_group;
   extern __shared__ int sh[];  // [experts] counts, [experts] first slots, [experts] cursors
   int* count = sh;
   int* first = sh + experts;
@@ -356,16 +370,24 @@ __global__ __launch_bounds__(1024) void expert_sort_kernel(const int* __restrict
   }
 }
 
-TK_API int tk_expert_sort(const int* ids, int pairs, int top, int experts, int max_tiles, int tm, int* slot_pair, int* slot_token,
-                          int* tile_group, hipStream_t stream) {
-  TK_REQUIRE(ids && slot_pair && slot_token && tile_group && pairs >= 0 && top > 0 && experts > 0, "expert_sort: bad arguments");
-  TK_REQUIRE(tm == GG_TM || tm == GS_M, "expert_sort: tiles of %d slots", tm);
-  TK_REQUIRE(max_tiles >= (pairs + tm - 1) / tm + experts, "expert_sort: %d tiles cannot hold %d pairs of %d experts", max_tiles,
-             pairs, experts);
-  TK_REQUIRE(3 * experts * sizeof(int) <= 48 * 1024, "expert_sort: too many experts");
-  hipLaunchKernelGGL(expert_sort_kernel, dim3(1), dim3(1024), 3 * experts * sizeof(int), stream, ids, pairs, top, experts,
-                     max_tiles, tm, slot_pair, slot_token, tile_group);
-  TK_CHECK_LAUNCH("expert_sort");
+TK_API int tk_expert_sort(const SortJob* jobs, int n_jobs, hipStream_t stream) {
+  TK_REQUIRE(jobs && n_jobs >= 0, "expert_sort: bad arguments");
+  for (int first = 0; first < n_jobs; first += SORT_JOBS) {
+    SortJobs all{};
+    const int n = min(SORT_JOBS, n_jobs - first);
+    int most = 0;
+    for (int k = 0; k < n; ++k) {
+      const SortJob& j = all.job[k] = jobs[first + k];
+      TK_REQUIRE(j.ids && j.slot_pair && j.slot_token && j.tile_group && j.pairs >= 0 && j.top > 0 && j.experts > 0, "expert_sort: bad arguments");
+      TK_REQUIRE(j.tm == GG_TM || j.tm == GS_M, "expert_sort: tiles of %d slots", j.tm);
+      TK_REQUIRE(j.max_tiles >= (j.pairs + j.tm - 1) / j.tm + j.experts, "expert_sort: %d tiles cannot hold %d pairs of %d experts", j.max_tiles,
+                 j.pairs, j.experts);
+      TK_REQUIRE(3 * j.experts * sizeof(int) <= 48 * 1024, "expert_sort: too many experts");
+      most = max(most, j.experts);
+    }
+    hipLaunchKernelGGL(expert_sort_kernel, dim3(n), dim3(1024), 3 * most * sizeof(int), stream, all);
+    TK_CHECK_LAUNCH("expert_sort");
+  }
   return 0;
 }
 

@@ -95,7 +95,7 @@ _SIGNATURES: dict[str, dict[str, list]] = {
         "tk_gemm_skinny_parts": [c_int, c_int, c_int],
         "tk_grouped_gemm_bf16": [_P, c_int, _P, _P, _P, c_int, c_int, c_int, c_int, _P, c_size_t, _P, c_int, c_int, c_int, c_int,
                                  c_int, c_int, _P, _P, c_int, c_float, c_float, _P],
-        "tk_expert_sort": [_P, c_int, c_int, c_int, c_int, c_int, _P, _P, _P, _P],
+        "tk_expert_sort": [_P, c_int, _P],
         "tk_expert_sum": [_P, c_int, _P, _P, _P, _P, _P, _P, c_int, c_int, c_int, c_int, c_int, _P],
     },
     "library": {

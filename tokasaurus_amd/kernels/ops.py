@@ -12,7 +12,6 @@ from dataclasses import dataclass
 
 import torch
 
-from tokasaurus_amd.kernels import lanes
 from tokasaurus_amd.kernels.library import KernelError, call, load
 
 _DT = {torch.float32: 0, torch.bfloat16: 1}
@@ -467,14 +466,17 @@ def attention_mfma_supports(dtype: torch.dtype, head_dim: int, page_size: int) -
 
 
 def check_attention_shape(dtype: torch.dtype, nq: int, nkv: int, head_dim: int, page_size: int,
-                          value_dim: int | None = None, generic_only: bool = False) -> None:
+                          value_dim: int | None = None, generic_only: bool = False, tile: bool = False) -> None:
     """Refuse, with the kernel's own reason, head counts and sizes that neither attention
     kernel takes for this storage type and page size.  Called when a cache is made for a
     mixer, so that a model that cannot run is refused before its first step.  ``generic_only``:
-    the mixer uses what only the 32-bit-arithmetic kernel has (a value size of its own, sinks)."""
+    the mixer uses what only the 32-bit-arithmetic kernel has (a value size of its own, sinks).  ``tile``: it takes the
+    32-bit matrix-core kernel where that takes the sizes."""
     vd = head_dim if value_dim is None else value_dim
     key_pages_shape(1, nkv, page_size, head_dim, padded=generic_only)
     value_pages_shape(1, nkv, page_size, vd)
+    if tile and attention_tile_f32_fits(nq, nkv, head_dim, vd, page_size):
+        return
     if generic_only or vd != head_dim or not attention_mfma_supports(dtype, head_dim, page_size):
         call("tk_paged_attention_generic_fits", nq, nkv, head_dim, vd)
 
@@ -1058,18 +1060,16 @@ def add(x: torch.Tensor, y: torch.Tensor) -> torch.Tensor:
 # What the product library's kernels may use for partial sums: its stream-K kernels want up to 64 MB
 # (one 256 x 256 tile of 32-bit sums a compute unit); the tensor library gives its products 76 MB too.
 LIBRARY_WORKSPACE_BYTES = 76 << 20
-_library_workspace: dict[tuple[int, int], torch.Tensor] = {}
+_library_workspace: dict[int, torch.Tensor] = {}
 
 
 def library_workspace() -> torch.Tensor:
     """The current device's workspace for library products: made at the first call (a runner
-    makes it before it records steps, so that no recording allocates it) and kept; one a lane
-    (``kernels.lanes``), for calls that run at the same time."""
+    makes it before it records steps, so that no recording allocates it) and kept."""
     device = torch._C._cuda_getDevice()
-    key = (device, lanes.lane())
-    ws = _library_workspace.get(key)
+    ws = _library_workspace.get(device)
     if ws is None:
-        ws = _library_workspace[key] = torch.empty(LIBRARY_WORKSPACE_BYTES, dtype=torch.uint8, device=f"cuda:{device}")
+        ws = _library_workspace[device] = torch.empty(LIBRARY_WORKSPACE_BYTES, dtype=torch.uint8, device=f"cuda:{device}")
     return ws
 
 
@@ -2216,15 +2216,60 @@ def expert_lookup(token_ids: torch.Tensor, last_token: torch.Tensor | None, tabl
     return [ids[at * n : (at + top) * n].view(n, top) for top, at in tables.spans]
 
 
+class _SortJob(ctypes.Structure):
+    """One choice to be sorted by expert (struct SortJob of grouped_gemm.hip)."""
+
+    _fields_ = [("ids", ctypes.c_void_p), ("slot_pair", ctypes.c_void_p), ("slot_token", ctypes.c_void_p), ("tile_group", ctypes.c_void_p),
+                ("pairs", ctypes.c_int), ("top", ctypes.c_int), ("experts", ctypes.c_int), ("max_tiles", ctypes.c_int), ("tm", ctypes.c_int)]
+
+
+@dataclass
+class SortedPairs:
+    """The pairs (token, place) of a choice sorted by expert into slots, tile by tile (see grouped_gemm.hip)."""
+
+    slot_pair: torch.Tensor
+    slot_token: torch.Tensor
+    tile_group: torch.Tensor
+    tile: int
+    max_tiles: int
+    shape: tuple  # of the ids
+
+
+def expert_sort(choices: "list[tuple[torch.Tensor, int]]") -> "list[SortedPairs]":
+    """(ids [tokens, top], number of experts) of one or several choices -> their pairs sorted, in one launch."""
+    out, jobs = [], (_SortJob * len(choices))()
+    for job, (ids, experts) in zip(jobs, choices):
+        _gpu(ids)
+        _i32(ids, "ids")
+        n, top = ids.shape
+        tile = GROUPED_LARGE_TILE if n * top >= GROUPED_LARGE_FROM * experts else GROUPED_TILE
+        max_tiles = -(-(n * top) // tile) + experts
+        slots = max_tiles * tile
+        book = torch.empty((2 * slots + max_tiles + 1,), dtype=torch.int32, device=ids.device)
+        s = SortedPairs(book[:slots], book[slots : 2 * slots], book[2 * slots :], tile, max_tiles, (n, top))
+        job.ids, job.slot_pair, job.slot_token, job.tile_group = (t.data_ptr() for t in (ids, s.slot_pair, s.slot_token, s.tile_group))
+        job.pairs, job.top, job.experts, job.max_tiles, job.tm = n * top, top, int(experts), max_tiles, tile
+        out.append(s)
+    call("tk_expert_sort", ctypes.addressof(jobs), len(choices), _stream())
+    return out
+
+
+def experts_go_in_tiles(rows: int, dtype: torch.dtype, width: int, ff: int) -> bool:
+    """Whether ``expert_mix`` sorts the pairs of so many tokens and runs the experts' products in tiles on the matrix cores
+    (for contiguous rows and weights)."""
+    return rows > GROUPED_FROM_ROWS and dtype == torch.bfloat16 and width % 8 == 0 and ff % 8 == 0
+
+
 def expert_mix(h: torch.Tensor, w_gate_up: torch.Tensor, w_down: torch.Tensor, ids: torch.Tensor, weights: torch.Tensor | None,
                shared: torch.Tensor | None = None, shared_gate: torch.Tensor | None = None,
-               weights_on_input: bool = False, glu: "tuple[float, float] | None" = None) -> torch.Tensor:
+               weights_on_input: bool = False, glu: "tuple[float, float] | None" = None, pairs: SortedPairs | None = None) -> torch.Tensor:
     """The weighted sum of a token's chosen experts, 32-bit [tokens, width]: expert e is
     ``w_down[e] (silu(gate) * up)`` with [gate | up] = ``w_gate_up[e] h``; an id from
     ``len(w_down)`` on names an identity expert (its output is h), a negative id an empty
     place.  ``shared`` (32-bit [tokens, width]) times ``shared_gate`` [tokens] is added.  ``weights_on_input``: a chosen
     expert reads weight * h and its output is added as it is (the factor goes on the 32-bit sums of gate and up).  ``glu``:
-    (limit, alpha) of the gated activation with clamps, in place of silu(gate) * up.  ``weights`` None: equal parts."""
+    (limit, alpha) of the gated activation with clamps, in place of silu(gate) * up.  ``weights`` None: equal parts.
+    ``pairs``: these very ids sorted by ``expert_sort`` (None: they are sorted here where it is wanted)."""
     _need(weights is not None or not weights_on_input, "expert_mix: equal parts multiply the experts' outputs")
     limit, alpha = (0.0, 0.0) if glu is None else (float(glu[0]), float(glu[1]))
     _need(glu is None or limit > 0.0, "expert_mix: the clamps' limit must be positive")
@@ -2250,13 +2295,11 @@ def expert_mix(h: torch.Tensor, w_gate_up: torch.Tensor, w_down: torch.Tensor, i
         return out
     if n > GROUPED_FROM_ROWS and _grouped_takes(h, w_gate_up, width) and ff % 8 == 0 and w_down.data_ptr() % 16 == 0:
         # many tokens: the pairs sorted by expert, every expert's rows in tiles on the matrix cores
-        tile = GROUPED_LARGE_TILE if n * top >= GROUPED_LARGE_FROM * experts else GROUPED_TILE
-        max_tiles = -(-(n * top) // tile) + experts
+        if pairs is None:
+            pairs = expert_sort([(ids, experts)])[0]
+        _need(pairs.shape == (n, top), "expert_mix: pairs of another choice")
+        slot_pair, slot_token, tile_group, tile, max_tiles = pairs.slot_pair, pairs.slot_token, pairs.tile_group, pairs.tile, pairs.max_tiles
         slots = max_tiles * tile
-        book = torch.empty((2 * slots + max_tiles + 1,), dtype=torch.int32, device=h.device)
-        slot_pair, slot_token, tile_group = book[:slots], book[slots : 2 * slots], book[2 * slots :]
-        call("tk_expert_sort", ids.data_ptr(), n * top, top, experts, max_tiles, tile, slot_pair.data_ptr(), slot_token.data_ptr(),
-             tile_group.data_ptr(), _stream())
         inter = torch.empty((slots, ff), dtype=h.dtype, device=h.device)
         call("tk_grouped_gemm_bf16", h.data_ptr(), h.stride(0), slot_token.data_ptr(), None, tile_group.data_ptr(), max_tiles, 0,
              0, 0, w_gate_up.data_ptr(), 2 * ff * width, inter.data_ptr(), ff, ff, width, slots, 1, 0, on_input,

@@ -208,8 +208,8 @@ class GroupedAttention(Mixer):
                          0 if self.value_dim == self.key_dim else self.value_dim, self.section)
 
     def check_cache(self, page_size: int, dtype: torch.dtype) -> None:
-        ops.check_attention_shape(dtype, self.num_heads, self.num_kv_heads, self.key_dim, page_size,
-                                  value_dim=self.value_dim, generic_only=True)
+        ops.check_attention_shape(dtype, self.num_heads, self.num_kv_heads, self.key_dim, page_size, value_dim=self.value_dim,
+                                  generic_only=True, tile=True)
 
     def load(self, tensors: dict[str, torch.Tensor], placer: Placer) -> None:
         self.qkv.load(tensors, placer)

@@ -6,7 +6,9 @@ the matrices side by side, ``[W_o left | W_o right]``, whose 32-bit sums are the
 mixers' results.  Or (``out_norms``) each mixer's own output, the full width, passes an RMS norm with a plain weight
 before the two are summed: ``left_scale * (rms_norm(left(h)) * w_left + rms_norm(right(h)) * w_right)``, both scales being
 equal; the two output projections are then products of their own, whose 32-bit sums a block may norm, sum and add to its
-stream in one pass (``normed_sum``), and in steps of many rows the two mixers run at the same time.  At most one of the two keeps keys in pages and at most one a state in the request's slot.
+stream in one pass (``normed_sum``).  The two run one after the other on the step's stream: their products share the library's
+handle and workspace, and some of its kernels wait for workgroups of their own that a second product may keep from starting.
+At most one of the two keeps keys in pages and at most one a state in the request's slot.
 """
 
 from __future__ import annotations
@@ -14,12 +16,8 @@ from __future__ import annotations
 import torch
 
 from tokasaurus_amd.kernels import ops
-from tokasaurus_amd.kernels.lanes import beside, join
 from tokasaurus_amd.parts.base import MIXERS, NORM_WEIGHT, CacheNeed, Mixer, NormedSum, Part, PartSpec, StateNeed, TensorSpec
 from tokasaurus_amd.parts.linear import Linear, Placer
-
-
-BESIDE_FROM_ROWS = 256
 
 
 @MIXERS.register("mixer_pair")
@@ -89,15 +87,7 @@ class MixerPair(Mixer):
             y = m.inner_rows(h, ctx, cache if m.cache_need() is not None else None, state if m.state_need() is not None else None)
             return m.out(y if rows is None else ops.gather_rows(y, rows), out_f32=True)
 
-        # steps of many rows: the two at the same time, for neither fills the chip (a recurrence is few long walks).  Recorded
-        # steps are left in one line: there the branches' hand-overs cost what they save.
-        if h.shape[0] >= BESIDE_FROM_ROWS and not ctx.extras.get("static"):
-            with beside():
-                right = branch(self.right)
-            left = branch(self.left)
-            join()
-        else:
-            left, right = branch(self.left), branch(self.right)
+        left, right = branch(self.left), branch(self.right)
         return NormedSum(left, self.norm_w[0], right, self.norm_w[1], float(self.out_norms["eps"]), self.left_scale)
 
     def mix(self, h, ctx, cache, state, rows, out_f32: bool = False):

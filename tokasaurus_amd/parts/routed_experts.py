@@ -130,23 +130,26 @@ class RoutedExperts(_Experts):
 
 class TokenTables:
     """The tables of a model's layers whose experts go by token id: they are read once a step, for all layers, in front
-    of the embedding."""
+    of the embedding, and the choices sorted by expert there too where the layers' products want that."""
 
-    KEY = "experts_by_token"  # in ``StepContext.extras``: per table the step's ids [tokens, top]
+    KEY = "experts_by_token"  # in ``StepContext.extras``: per table the step's ids [tokens, top] and, or None, their sorted pairs
 
     def __init__(self):
-        self.tables: list[torch.Tensor] = []
+        self.layers: list[TableExperts] = []
         self._ready: "ops.ExpertTables | None" = None
 
-    def add(self, table: torch.Tensor) -> int:
-        self.tables.append(table)
+    def add(self, layer: "TableExperts") -> int:
+        self.layers.append(layer)
         self._ready = None
-        return len(self.tables) - 1
+        return len(self.layers) - 1
 
     def __call__(self, ctx: StepContext) -> None:
         if self._ready is None:
-            self._ready = ops.ExpertTables(self.tables)
-        ctx.extras[self.KEY] = ops.expert_lookup(ctx.token_ids, ctx.last_token, self._ready)
+            self._ready = ops.ExpertTables([x.table for x in self.layers])
+        ids = ops.expert_lookup(ctx.token_ids, ctx.last_token, self._ready)
+        tiled = [i for i, x in enumerate(self.layers) if ops.experts_go_in_tiles(ctx.num_tokens, ctx.dtype, x.hidden_size, x.expert_size)]
+        made = dict(zip(tiled, ops.expert_sort([(ids[i], self.layers[i].num_experts) for i in tiled]))) if tiled else {}
+        ctx.extras[self.KEY] = [(x, made.get(i)) for i, x in enumerate(ids)]
 
 
 @FEED_FORWARDS.register("table_experts")
@@ -168,6 +171,7 @@ class TableExperts(_Experts):
             shared["token_tables"] = TokenTables()
             shared.setdefault("step_starts", []).append(shared["token_tables"])
         self.tables: TokenTables = shared["token_tables"]
+        self.table: torch.Tensor | None = None
         self.index: int | None = None
 
     def tensor_specs(self) -> list[TensorSpec]:
@@ -176,13 +180,14 @@ class TableExperts(_Experts):
     def load(self, tensors: dict[str, torch.Tensor], placer: Placer) -> None:
         self._load_experts(tensors, placer)
         name = self.names["table"]
-        self.index = self.tables.add(placer.place(("int_table", name), lambda: tensors[name].to(torch.int32).contiguous().to(placer.device)))
+        self.table = placer.place(("int_table", name), lambda: tensors[name].to(torch.int32).contiguous().to(placer.device))
+        self.index = self.tables.add(self)
 
     def transform(self, h: torch.Tensor, out_f32: bool = False, ctx: StepContext | None = None, rows: torch.Tensor | None = None):
-        ids = ctx.extras[TokenTables.KEY][self.index]
+        ids, pairs = ctx.extras[TokenTables.KEY][self.index]
         if rows is not None:
-            ids = ids.index_select(0, rows)
-        y = ops.expert_mix(h, self.w_gate_up, self.w_down, ids, None, glu=self.glu)
+            ids, pairs = ids.index_select(0, rows), None
+        y = ops.expert_mix(h, self.w_gate_up, self.w_down, ids, None, glu=self.glu, pairs=pairs)
         return y if out_f32 else y.to(h.dtype)
 
     def forward(self, h: torch.Tensor, residual: torch.Tensor, ctx: StepContext | None = None, rows: torch.Tensor | None = None):
