@@ -2100,7 +2100,7 @@ def squared_relu_(x: torch.Tensor) -> torch.Tensor:
 GROUPED_TILE = 64  # slots a tile of the grouped matrix-core product (GG_TM of grouped_gemm.hip)
 GROUPED_LARGE_TILE = 128  # of the one that goes through local memory (GS_M)
 GROUPED_LARGE_FROM = 96  # pairs an expert has on average from which on the experts' products take the large tiles
-GROUPED_FROM_ROWS = 16  # rows above which the products of experts and of heads run in tiles on the matrix cores
+GROUPED_FROM_ROWS = 12  # rows above which the products of experts and of heads run in tiles on the matrix cores
 
 
 def _grouped_takes(x: torch.Tensor, w: torch.Tensor, inner: int) -> bool:
